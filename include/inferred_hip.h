@@ -102,6 +102,7 @@ enum {
     IT_HIP_NO_GRAPH = 2, /* never capture decode passes into a HIP graph */
     IT_HIP_NO_FUSE = 4,  /* capture decode passes op by op, without the fused kernels */
     IT_HIP_NO_CHAIN = 8, /* keep every fused decode stage a launch of its own (no persistent kernel over runs of layers) */
+    IT_HIP_F32 = 16, /* models with unquantized matrices: 32-bit throughout (no half-precision products, caches of f32) */
 };
 
 /* Cuda::new, src/ops/cuda/mod.rs:757-935.  NULL on failure with a message in err. */
@@ -315,6 +316,79 @@ void it_hip_zero_state(it_hip*);
  * (2 per multiply-accumulate).  0 = ok, 1 = bad argument, 2 = device error */
 int it_hip_mfma_ceiling(it_hip*, int kind, int iters, double* ops_per_s);
 
+/* ---- ops of models with unquantized matrices (no counterpart in the reference's trait) ----
+ * Same conventions as the ops above: host pointers as names of device mirrors, resident weights and device-owned slabs;
+ * batch size from the buffer lengths; first error kept.  Each op is one sublayer step and picks its form by the batch: one
+ * token a fused launch, up to 16 tokens a few, more tokens the bf16 matrix cores (bf16 matrices, and not in 32-bit mode:
+ * IT_HIP_F32 and IT_HIP_EXACT take 32-bit kernels throughout).  With IT_HIP_NO_FUSE every step of an op is a launch. */
+/* One matrix of a group that reads the same activations.  `up` (data non-NULL) makes it a gated pair: silu(w x) * (up x).
+ * The rows go to `out` (times `scale`), or, with `slab` set, to rows slab_row .. of a cache slab whose elements are f16 (f32
+ * in 32-bit mode): heads of head_dim elements, head_stride elements apart, n_out / head_dim of them a row. */
+typedef struct {
+    it_weights w, up;
+    float* out;
+    uint64_t out_len;
+    void* slab;
+    uint64_t slab_len; /* elements */
+    uint64_t slab_row, head_dim, head_stride;
+    float scale;
+    uint32_t _pad;
+} it_group_mat;
+/* out_m = scale_m * W_m h, h = RMS norm of x times norm_w (norm_w NULL: h = x); at most 6 matrices of n_in = row length */
+void it_hip_norm_matmuls(it_hip*, const float* x, uint64_t x_len, const float* norm_w, uint64_t n_in, float eps,
+                         const it_group_mat* mats, uint64_t n_mats);
+/* One term of a residual sum: scale (elementwise, NULL: 1) times W applied to `in`, whose rows are first, when norm_w is
+ * set, cut into norm_groups equal parts, each divided by its own root mean square, and multiplied by norm_w. */
+typedef struct {
+    it_weights w;
+    const float* in;
+    uint64_t in_len;
+    const float* scale;
+    const float* norm_w;
+    uint64_t norm_groups;
+    float eps;
+    uint32_t _pad;
+} it_res_term;
+/* x += sum of at most 2 terms; the terms are added up before x is */
+void it_hip_matmul_residual(it_hip*, float* x, uint64_t x_len, const it_res_term* terms, uint64_t n_terms);
+/* Causal attention of the last n_q of n_pos positions over slabs written by it_hip_norm_matmuls:
+ *   score = (q . k) * scale * temp(position) - slopes[head] * (position - key), slopes NULL: no bias;
+ *   temp(p) = 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1), temp_coef 0: none;
+ *   weights = exp(score) / (sink + sum exp(score)), sink 0 or 1; query head h reads KV head h / (n_head / n_head_kv) */
+typedef struct {
+    const float* q;
+    uint64_t q_len;
+    const void *k, *v;
+    uint64_t k_len, v_len; /* elements in each slab */
+    uint64_t n_pos, k_dim, v_dim, k_stride, v_stride, n_head, n_head_kv;
+    float scale;
+    uint32_t sink;
+    const float* slopes;
+    float temp_coef;
+    uint32_t temp_every;
+} it_attn_bias;
+void it_hip_attend_bias(it_hip*, const it_attn_bias* a, float* out, uint64_t out_len);
+/* The Mamba-2 mixer between its projections: u rows are [z | x | B | C | dt] (inner, inner, groups * n, groups * n, heads;
+ * inner = heads * vdim); out rows are the gated read-out y * silu(z) of `inner` floats, not yet normed.
+ * conv_ring: taps rows of the x, B, C channels, row p % taps the raw input of position p; state: [heads][vdim][n].
+ * `pos` is the position of the first token. */
+typedef struct {
+    const float *conv_w, *conv_b, *dt_bias, *a_log, *d;
+    uint64_t heads, vdim, n, groups, taps, pos;
+} it_mamba2;
+void it_hip_mamba2(it_hip*, const it_mamba2* m, const float* u, uint64_t u_len, float* conv_ring, uint64_t ring_len, float* state,
+                   uint64_t state_len, float* out, uint64_t out_len);
+/* x[t] += rows[t] (NULL: none), then + vec (NULL: none) */
+void it_hip_add_rows(it_hip*, float* x, uint64_t x_len, const float* rows, const float* vec, uint64_t vec_len);
+/* out = the rows `idx` of src (rows of `width` floats) */
+void it_hip_gather_rows(it_hip*, const float* src, uint64_t src_len, uint64_t width, const uint32_t* idx, uint64_t n_rows, float* out,
+                        uint64_t out_len);
+/* 1 when this backend keeps caches of unquantized models in f32 */
+int it_hip_is_f32(const it_hip*);
+/* the caller has zeroed the host copy of ONE recurrent-state slab: its device copy is zeroed in place (it_hip_zero_state
+ * does this for every slab of the backend, which is too much where several sequences share it) */
+void it_hip_zero_slab(it_hip*, const void* host);
+
 /* ---- one entry point that allocates nothing ----
  * No counterpart in the reference (its device backend sizes its pools with the driver's allocator as it goes,
  * src/ops/cuda/mod.rs:1011-1158).  For callers that cannot allocate: code under HIP graph capture, tight serving
@@ -342,7 +416,9 @@ typedef struct it_model it_model;
 typedef struct it_engine it_engine;
 typedef void (*it_trace_fn)(void* user, const char* name, uint32_t layer, const float* data, uint64_t n);
 
-it_model* it_model_open(const char* gguf_path, char* err, size_t err_len);
+/* `path`: a GGUF file (qwen35moe), or a folder with config.json and model.safetensors (Serisun); the design is chosen by the
+ * architecture name the file or the configuration gives */
+it_model* it_model_open(const char* path, char* err, size_t err_len);
 void it_model_close(it_model*);
 /* n_layer n_embd n_vocab n_head n_head_kv head_dim n_expert n_expert_used expert_ff n_rot */
 void it_model_dims(const it_model*, uint64_t out[10]);
@@ -369,6 +445,8 @@ int it_engine_rewind(it_engine*, uint64_t len);
 int it_engine_forward(it_engine*, const uint32_t* tokens, uint64_t n, float* logits);
 /* chunked prefill; logits of the last token (may be NULL) */
 int it_engine_prefill(it_engine*, const uint32_t* tokens, uint64_t n, float* logits);
+/* the same passes with the logits of the tokens `rows` (ascending indexes into `tokens`) to out [n_rows][n_vocab] */
+int it_engine_forward_rows(it_engine*, const uint32_t* tokens, uint64_t n, const uint32_t* rows, uint64_t n_rows, float* out);
 /* greedy generation; returns tokens produced or a negative error */
 int64_t it_engine_generate(it_engine*, const uint32_t* prompt, uint64_t n_prompt, uint64_t max_new,
                            uint32_t* out_ids, float* last_logits);

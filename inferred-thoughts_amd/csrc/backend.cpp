@@ -279,7 +279,7 @@ float* it_hip::act_in(const float* host, size_t len) {
         h2d++;
         h2d_bytes += len * sizeof(float);
         a->dev_current = true;
-        a->q_valid = false;
+        a->stale_forms();
     }
     return a->dev;
 }
@@ -288,7 +288,7 @@ float* it_hip::act_out(const float* host, size_t len) {
     if (!a) return nullptr;
     a->dev_current = true;
     a->elided = false;
-    a->q_valid = false;
+    a->stale_forms();
     return a->dev;
 }
 bool it_hip::held_touches(const void* dev, size_t bytes) const {
@@ -311,7 +311,7 @@ void it_hip::mark_elided(const std::vector<const void*>& devs) {
 }
 float* it_hip::act_inout(const float* host, size_t len) {
     float* d = act_in(host, len);
-    if (d) acts[host].q_valid = false;
+    if (d) acts[host].stale_forms();
     return d;
 }
 
@@ -1077,6 +1077,7 @@ void it_hip::drop_all() {
         if (kv.second.dev) (void)hipFree(kv.second.dev);
         if (kv.second.q_scales) (void)hipFree(kv.second.q_scales);
         if (kv.second.q_quants) (void)hipFree(kv.second.q_quants);
+        if (kv.second.h16) (void)hipFree(kv.second.h16);
     }
     acts.clear();
     for (auto& kv : consts)
@@ -1119,6 +1120,8 @@ it_hip::~it_hip() {
     if (route_w) (void)hipFree(route_w);
     if (attn_scratch) (void)hipFree(attn_scratch);
     if (gdn_work) (void)hipFree(gdn_work);
+    for (Tmp& t : tmps)
+        if (t.p) (void)hipFree(t.p);
     if (moe_f16) (void)hipFree(moe_f16);
     if (zero_ids) (void)hipFree(zero_ids);
     if (moe_work) (void)hipFree(moe_work);
@@ -1229,6 +1232,7 @@ it_hip* it_hip_create(uint32_t flags, int device, char* err, size_t err_len) {
     it_hip* be = new it_hip();
     be->device = device;
     be->exact = (flags & IT_HIP_EXACT) != 0;
+    be->f32 = (flags & (IT_HIP_F32 | IT_HIP_EXACT)) != 0;
     be->allow_graph = (flags & IT_HIP_NO_GRAPH) == 0;
     be->fuse_enabled = (flags & IT_HIP_NO_FUSE) == 0 && getenv("INFERRED_HIP_NO_FUSE") == nullptr;
     be->chain_enabled = (flags & IT_HIP_NO_CHAIN) == 0 && getenv("INFERRED_HIP_NO_CHAIN") == nullptr;
@@ -2053,7 +2057,7 @@ void it_hip_host_wrote(it_hip* be, const float* buf, uint64_t len) {
     auto it = be->acts.find(buf);
     if (it != be->acts.end()) {
         it->second.dev_current = false;
-        it->second.q_valid = false;
+        it->second.stale_forms();
     }
 }
 
@@ -2114,7 +2118,7 @@ void it_hip_begin_pass(it_hip* be, uint64_t n_tokens) {
     for (auto& kv : be->acts) {
         kv.second.dev_current = false;
         kv.second.elided = false;
-        kv.second.q_valid = false;
+        kv.second.stale_forms();
     }
 }
 
@@ -2434,6 +2438,10 @@ void it_hip_release(it_hip* be, const void* host) {
         if (a->second.dev) (void)hipFree(a->second.dev);
         if (a->second.q_scales) (void)hipFree(a->second.q_scales);
         if (a->second.q_quants) (void)hipFree(a->second.q_quants);
+        if (a->second.h16) {
+            be->quant_bytes -= a->second.h_cap * sizeof(uint16_t);
+            (void)hipFree(a->second.h16);
+        }
         be->acts.erase(a);
     }
     if (s != be->slabs.end()) {
@@ -2476,7 +2484,9 @@ int it_hip_profile_end(it_hip* be, it_profile_row* rows, int max_rows) {
                                                    "norms", "router (softmax + top-k)", "other",
                                                    "fused_gemv (norm + quantize + dense GEMVs)", "lm_head (norm + GEMV)",
                                                    "gdn_rows (l2 norm + delta rule)", "attn_prep (norm + rope + kv write)",
-                                                   "layer_chain (a run of layers, persistent)"};
+                                                   "layer_chain (a run of layers, persistent)",
+                                                   "group (norm + unquantized matrices)",
+                                                   "residual (matrices + residual sum)", "mamba2 (conv + state space)"};
     be->prof_on = false;
     be->check(hipStreamSynchronize(be->stream), "sync");
     it_profile_row acc[it_hip::FAM_COUNT];

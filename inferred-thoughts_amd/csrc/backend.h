@@ -19,6 +19,7 @@
 
 #include "../../include/inferred_hip.h"
 #include "kernels.h"
+#include "kernels_float.h"
 #include "kernels_fused.h"
 
 // Seam ops as recorded for the fuser.  Pointer/int slots per op:
@@ -43,12 +44,14 @@
 enum OpId : int {
     OP_RMS = 1, OP_RMS_HEADS, OP_L2, OP_MATMUL, OP_ROPE, OP_SOFTMAX, OP_ATTEND, OP_EW, OP_SCALE, OP_CONV, OP_GATHER,
     OP_SCATTER, OP_DELTA, OP_ROUTE, OP_EXPERTS, OP_GLU, OP_FINISH, OP_ROWS, OP_SIGADD, OP_KVWRITE, OP_EMBED,
+    OP_GROUP, OP_RESIDUAL, OP_ATTEND_BIAS, OP_MAMBA2, OP_ADD_ROWS, OP_GATHER_ROWS,   // unquantized models: issued as they are
     OP_QUANT = 101
 };
 
 struct it_hip {
     // ---- configuration
     bool exact = false;
+    bool f32 = false;   // unquantized models in 32-bit throughout (exact mode implies it for them)
     bool allow_graph = true;
     int device = 0;
     hipStream_t stream = nullptr;
@@ -71,6 +74,12 @@ struct it_hip {
         size_t q_cap = 0;  // floats covered
         size_t q_len = 0;
         bool q_valid = false;
+        // bf16 form of rows of h_row floats (each padded to a multiple of 8), for products on the bf16 matrix cores
+        uint16_t* h16 = nullptr;
+        size_t h_cap = 0;      // elements
+        size_t h_rows = 0, h_row = 0;
+        bool h_valid = false;
+        void stale_forms() { q_valid = h_valid = false; }
     };
     std::unordered_map<const void*, Act> acts;
     Act* act_slot(const float* host, size_t len);
@@ -80,6 +89,14 @@ struct it_hip {
     bool act_quantized(const float* host, size_t len, const float** scales, const int8_t** quants,
                        float** dev_x);
     bool act_q_reserve(Act& a, size_t len);  // room for the Q8_0 form of `len` floats
+    // the bf16 form about to be written by the op that produces the rows (the f32 mirror keeps stale bytes: elided)
+    uint16_t* act_half_out(const float* host, size_t rows, size_t row);
+    uint16_t* act_half_reserve(Act& a, size_t rows, size_t row);
+    const uint16_t* act_half_if_valid(const float* host, size_t rows, size_t row);
+    // scratch of the unquantized ops, by use: f32 rows, bf16 rows
+    struct Tmp { void* p = nullptr; size_t bytes = 0; };
+    Tmp tmps[6];
+    void* tmp_for(int which, size_t bytes);
     Act* act_by_dev(const void* dev);        // the mirror whose device buffer holds `dev`, or null
     bool held_touches(const void* dev, size_t bytes) const;   // an op held back reads or writes inside [dev, dev + bytes)
     // marks the mirrors at these device addresses as not holding their ops' values (a fused kernel skipped the writes):
@@ -348,7 +365,7 @@ struct it_hip {
 
     // ---- per-kernel-family timing with HIP events on the launch stream
     enum Family { FAM_MATMUL = 0, FAM_MOE_GLU, FAM_MOE_DOWN, FAM_DELTA, FAM_ATTEND, FAM_NORM, FAM_ROUTER, FAM_OTHER,
-                  FAM_FUSED_GEMV, FAM_LM_HEAD, FAM_GDN_ROWS, FAM_ATTN_PREP, FAM_CHAIN, FAM_COUNT };
+                  FAM_FUSED_GEMV, FAM_LM_HEAD, FAM_GDN_ROWS, FAM_ATTN_PREP, FAM_CHAIN, FAM_GROUP, FAM_RESIDUAL, FAM_SSD, FAM_COUNT };
     struct ProfSpan {
         hipEvent_t a, b;
         int fam;

@@ -1,0 +1,537 @@
+// Products of several unquantized matrices with the same activations (a norm's output feeding the query, key, value,
+// gate and up projections of a parallel layer), and sums of products added to the residual stream.
+//
+// One token (decode): a launch per group.  Every block forms the normed input in LDS while its first weight rows are
+// in flight; a wave then takes groups of R rows, 16 bytes of each row a lane, and finishes them where they belong:
+// f32 rows, cache slabs, or silu(gate) * up.  Activations stay f32 throughout, so the arithmetic is the same in
+// 32-bit mode.  A few tokens: one weight row a wave, eight tokens a pass.  Many tokens take k_gemm_bf16.hip.
+#include "it_device.h"
+#include "it_float.h"
+#include "it_reduce.h"
+#include "kernels_float.h"
+
+namespace itk {
+namespace {
+
+constexpr int CH = 512;   // elements of a row a wave takes at a time, eight a lane
+
+template <int FMT> struct Raw8 { uint4 a; };
+template <> struct Raw8<W_F32> { uint4 a, b; };
+
+template <int FMT> IT_DEV const uint8_t* row_at(const uint8_t* w, int64_t row, int n_in) {
+    return w + row * n_in * (FMT == W_F32 ? 4 : 2);
+}
+// eight elements of a row from k on; AL: the row length is a multiple of 8 and the rows are 16-byte aligned
+template <int FMT, bool AL> IT_DEV Raw8<FMT> load8(const uint8_t* row, int k, int n_in) {
+    Raw8<FMT> r{};
+    if (AL) {
+        if (k < n_in) {
+            if constexpr (FMT == W_F32) {
+                r.a = *(const uint4*)((const float*)row + k);
+                r.b = *(const uint4*)((const float*)row + k + 4);
+            } else {
+                r.a = *(const uint4*)((const uint16_t*)row + k);
+            }
+        }
+    } else {
+        uint32_t v[8];
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+            if (FMT == W_F32) v[e] = k + e < n_in ? ((const uint32_t*)row)[k + e] : 0u;
+            else v[e] = k + e < n_in ? ((const uint16_t*)row)[k + e] : 0u;
+        }
+        if constexpr (FMT == W_F32) {
+            r.a = make_uint4(v[0], v[1], v[2], v[3]);
+            r.b = make_uint4(v[4], v[5], v[6], v[7]);
+        } else {
+            r.a = make_uint4(v[0] | (v[1] << 16), v[2] | (v[3] << 16), v[4] | (v[5] << 16), v[6] | (v[7] << 16));
+        }
+    }
+    return r;
+}
+template <int FMT> IT_DEV void widen8(const Raw8<FMT>& r, float* f) {
+    if constexpr (FMT == W_F32) {
+        const uint32_t v[8] = {r.a.x, r.a.y, r.a.z, r.a.w, r.b.x, r.b.y, r.b.z, r.b.w};
+#pragma unroll
+        for (int e = 0; e < 8; e++) f[e] = __uint_as_float(v[e]);
+    } else {
+        const uint32_t v[4] = {r.a.x, r.a.y, r.a.z, r.a.w};
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            if (FMT == W_BF16) {
+                f[2 * e] = __uint_as_float(v[e] << 16);
+                f[2 * e + 1] = __uint_as_float(v[e] & 0xffff0000u);
+            } else {
+                f[2 * e] = it_f16_to_f32((uint16_t)(v[e] & 0xffffu));
+                f[2 * e + 1] = it_f16_to_f32((uint16_t)(v[e] >> 16));
+            }
+        }
+    }
+}
+
+// which matrix a group of rows belongs to
+struct Groups {
+    int first[GROUP_MAX + 1];
+    int n;
+};
+
+IT_DEV float block_sum(float v, float* red) {   // 256 threads
+    v = group_sum<64>(v);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return (red[0] + red[1]) + (red[2] + red[3]);
+}
+
+constexpr int U = 4;   // row pieces of a wave in flight
+
+template <int FMT, bool AL, int R>
+__global__ __launch_bounds__(256) void group_gemv_k(GroupP p, Groups gs) {
+    extern __shared__ __align__(16) float xs[];   // the input, zero past its end to a whole number of pieces
+    __shared__ float red[4];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int n_ch = (p.n_in + CH - 1) / CH;
+    const uint8_t* rp[R];
+    Raw8<FMT> w[R][U];
+    int mi = 0, j0 = 0;
+    auto open = [&](int g) __attribute__((always_inline)) {
+        mi = 0;
+        while (mi + 1 < p.n_mats && g >= gs.first[mi + 1]) mi++;
+        const GroupMat& m = p.m[mi];
+        const int at = g - gs.first[mi];
+        if (m.up) {
+            j0 = at * (R / 2);
+#pragma unroll
+            for (int r = 0; r < R; r++) rp[r] = row_at<FMT>(r < R / 2 ? m.w : m.up, min(j0 + r % (R / 2), m.n_out - 1), p.n_in);
+        } else {
+            j0 = at * R;
+#pragma unroll
+            for (int r = 0; r < R; r++) rp[r] = row_at<FMT>(m.w, min(j0 + r, m.n_out - 1), p.n_in);
+        }
+    };
+    auto load = [&](int c0) __attribute__((always_inline)) {
+#pragma unroll
+        for (int u = 0; u < U; u++)
+#pragma unroll
+            for (int r = 0; r < R; r++) w[r][u] = load8<FMT, AL>(rp[r], (c0 + u) * CH + lane * 8, p.n_in);
+    };
+    int g = blockIdx.x * 4 + wave;
+    if (g < gs.n) {
+        open(g);
+        load(0);
+    }
+    // the input while the first rows are on their way
+    {
+        float ss = 0.0f;
+        for (int i = tid; i < n_ch * CH; i += 256) {
+            const float v = i < p.n_in ? p.x[i] : 0.0f;
+            ss = fmaf(v, v, ss);
+            xs[i] = v;
+        }
+        if (p.norm_w) {
+            ss = block_sum(ss, red);
+            const float rinv = 1.0f / sqrtf(ss / (float)p.n_in + p.eps);
+            for (int i = tid; i < p.n_in; i += 256) xs[i] = xs[i] * rinv * p.norm_w[i];
+        }
+        __syncthreads();
+    }
+    for (bool first = true; g < gs.n; g += gridDim.x * 4, first = false) {
+        if (!first) open(g);
+        float acc[R];
+#pragma unroll
+        for (int r = 0; r < R; r++) acc[r] = 0.0f;
+        for (int c0 = 0; c0 < n_ch; c0 += U) {
+            if (!first || c0 > 0) load(c0);
+#pragma unroll
+            for (int u = 0; u < U; u++) {
+                if (c0 + u < n_ch) {
+                    const float4 x0 = *(const float4*)(xs + (c0 + u) * CH + lane * 8), x1 = *(const float4*)(xs + (c0 + u) * CH + lane * 8 + 4);
+                    const float x[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
+#pragma unroll
+                    for (int r = 0; r < R; r++) {
+                        float f[8];
+                        widen8<FMT>(w[r][u], f);
+#pragma unroll
+                        for (int e = 0; e < 8; e++) acc[r] = fmaf(f[e], x[e], acc[r]);
+                    }
+                }
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < R; r++) acc[r] = group_sum<64>(acc[r]);
+        const GroupMat& m = p.m[mi];
+        // lane r finishes row r
+        if (m.up) {
+#pragma unroll
+            for (int r = 0; r < R / 2; r++)
+                if (lane == r && j0 + r < m.n_out) group_store(m, 0, j0 + r, silu_exact(acc[r]) * acc[R / 2 + r]);
+        } else {
+#pragma unroll
+            for (int r = 0; r < R; r++)
+                if (lane == r && j0 + r < m.n_out) group_store(m, 0, j0 + r, acc[r]);
+        }
+    }
+}
+
+// ---------------------------------------------------------------- one token: sum of products into the residual
+template <int FMT, bool AL, int R>
+__global__ __launch_bounds__(256) void res_gemv_k(ResP p) {
+    extern __shared__ __align__(16) float xs[];   // the terms' inputs one behind the other, each padded to whole pieces
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int j0 = (blockIdx.x * 4 + wave) * R;
+    Raw8<FMT> w[R][U];
+    auto load = [&](const ResTerm& t, int c0) __attribute__((always_inline)) {
+#pragma unroll
+        for (int u = 0; u < U; u++)
+#pragma unroll
+            for (int r = 0; r < R; r++) w[r][u] = load8<FMT, AL>(row_at<FMT>(t.w, min(j0 + r, p.n_out - 1), t.n_in), (c0 + u) * CH + lane * 8, t.n_in);
+    };
+    load(p.t[0], 0);
+    {
+        float* at = xs;
+        for (int k = 0; k < p.n_terms; k++) {
+            const int len = (p.t[k].n_in + CH - 1) / CH * CH;
+            for (int i = tid; i < len; i += 256) at[i] = i < p.t[k].n_in ? p.t[k].in[i] : 0.0f;
+            at += len;
+        }
+        __syncthreads();
+        at = xs;
+        for (int k = 0; k < p.n_terms; k++) {
+            const ResTerm& t = p.t[k];
+            if (t.norm_w) {
+                const int part = t.n_in / t.norm_groups;
+                for (int gi = wave; gi < t.norm_groups; gi += 4) {
+                    float ss = 0.0f;
+                    for (int i = lane; i < part; i += 64) ss = fmaf(at[gi * part + i], at[gi * part + i], ss);
+                    ss = group_sum<64>(ss);
+                    const float rinv = 1.0f / sqrtf(ss / (float)part + t.eps);
+                    for (int i = lane; i < part; i += 64) at[gi * part + i] = at[gi * part + i] * rinv * t.norm_w[gi * part + i];
+                }
+            }
+            at += (t.n_in + CH - 1) / CH * CH;
+        }
+        __syncthreads();
+    }
+    if (j0 >= p.n_out) return;
+    float total[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) total[r] = 0.0f;
+    const float* at = xs;
+    for (int k = 0; k < p.n_terms; k++) {
+        const ResTerm& t = p.t[k];
+        const int n_ch = (t.n_in + CH - 1) / CH;
+        float acc[R];
+#pragma unroll
+        for (int r = 0; r < R; r++) acc[r] = 0.0f;
+        for (int c0 = 0; c0 < n_ch; c0 += U) {
+            if (k > 0 || c0 > 0) load(t, c0);
+#pragma unroll
+            for (int u = 0; u < U; u++) {
+                if (c0 + u < n_ch) {
+                    const float4 x0 = *(const float4*)(at + (c0 + u) * CH + lane * 8), x1 = *(const float4*)(at + (c0 + u) * CH + lane * 8 + 4);
+                    const float x[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
+#pragma unroll
+                    for (int r = 0; r < R; r++) {
+                        float f[8];
+                        widen8<FMT>(w[r][u], f);
+#pragma unroll
+                        for (int e = 0; e < 8; e++) acc[r] = fmaf(f[e], x[e], acc[r]);
+                    }
+                }
+            }
+        }
+        at += n_ch * CH;
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            acc[r] = group_sum<64>(acc[r]);
+            total[r] += t.scale ? acc[r] * t.scale[min(j0 + r, p.n_out - 1)] : acc[r];
+        }
+    }
+#pragma unroll
+    for (int r = 0; r < R; r++)
+        if (lane == r && j0 + r < p.n_out) p.x[j0 + r] += total[r];
+}
+
+// ---------------------------------------------------------------- a few tokens
+constexpr int NT = 8;
+
+template <int FMT, bool AL>
+IT_DEV void dot_rows(const uint8_t* row, const float* x, int n_in, int n_tok, int t0, int lane, float* acc) {
+#pragma unroll
+    for (int t = 0; t < NT; t++) acc[t] = 0.0f;
+    for (int k = lane * 8; k < n_in; k += CH) {
+        float f[8];
+        widen8<FMT>(load8<FMT, AL>(row, k, n_in), f);
+#pragma unroll
+        for (int t = 0; t < NT; t++) {
+            if (t0 + t < n_tok) {
+                const float* xt = x + (int64_t)(t0 + t) * n_in + k;
+#pragma unroll
+                for (int e = 0; e < 8; e++)
+                    if (AL || k + e < n_in) acc[t] = fmaf(f[e], xt[e], acc[t]);
+            }
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < NT; t++) acc[t] = group_sum<64>(acc[t]);
+}
+
+template <int FMT, bool AL>
+__global__ __launch_bounds__(256) void group_rows_k(GroupP p, Groups gs) {   // a group is one row (one gate / up pair)
+    const int lane = threadIdx.x & 63, g = blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    if (g >= gs.n) return;
+    int mi = 0;
+    while (mi + 1 < p.n_mats && g >= gs.first[mi + 1]) mi++;
+    const GroupMat& m = p.m[mi];
+    const int j = g - gs.first[mi], t0 = blockIdx.y * NT;
+    float a[NT], b[NT];
+    dot_rows<FMT, AL>(row_at<FMT>(m.w, j, p.n_in), p.x, p.n_in, p.n_tok, t0, lane, a);
+    if (m.up) dot_rows<FMT, AL>(row_at<FMT>(m.up, j, p.n_in), p.x, p.n_in, p.n_tok, t0, lane, b);
+#pragma unroll
+    for (int t = 0; t < NT; t++)
+        if (lane == t && t0 + t < p.n_tok) group_store(m, t0 + t, j, m.up ? silu_exact(a[t]) * b[t] : a[t]);
+}
+
+template <int FMT, bool AL>
+__global__ __launch_bounds__(256) void res_rows_k(ResP p) {
+    const int lane = threadIdx.x & 63, j = blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    if (j >= p.n_out) return;
+    const int t0 = blockIdx.y * NT;
+    float total[NT], a[NT];
+#pragma unroll
+    for (int t = 0; t < NT; t++) total[t] = 0.0f;
+    for (int k = 0; k < p.n_terms; k++) {
+        const ResTerm& q = p.t[k];
+        dot_rows<FMT, AL>(row_at<FMT>(q.w, j, q.n_in), q.in, q.n_in, p.n_tok, t0, lane, a);
+        const float sc = q.scale ? q.scale[j] : 1.0f;
+#pragma unroll
+        for (int t = 0; t < NT; t++) total[t] += a[t] * sc;
+    }
+#pragma unroll
+    for (int t = 0; t < NT; t++)
+        if (lane == t && t0 + t < p.n_tok) p.x[(int64_t)(t0 + t) * p.n_out + j] += total[t];
+}
+
+// ---------------------------------------------------------------- norms, conversions, sums
+__global__ __launch_bounds__(256) void norm_rows_k(const float* __restrict__ x, const float* __restrict__ w, int groups, float eps,
+                                                   int nd, float* __restrict__ out32, uint16_t* __restrict__ out16) {
+    __shared__ float red[4];
+    const int part = nd / groups, g = blockIdx.y, tid = threadIdx.x;
+    const int64_t row = blockIdx.x;
+    const float* xr = x + row * nd + g * part;
+    float rinv = 1.0f;
+    if (w) {
+        float ss = 0.0f;
+        for (int i = tid; i < part; i += 256) ss = fmaf(xr[i], xr[i], ss);
+        ss = block_sum(ss, red);
+        rinv = 1.0f / sqrtf(ss / (float)part + eps);
+    }
+    for (int i = tid; i < part; i += 256) {
+        const float v = w ? xr[i] * rinv * w[g * part + i] : xr[i];
+        if (out32) out32[row * nd + g * part + i] = v;
+        if (out16) out16[row * pad8(nd) + g * part + i] = to_bf16(v);
+    }
+    if (out16 && g == groups - 1 && tid < pad8(nd) - nd) out16[row * pad8(nd) + nd + tid] = 0;
+}
+
+// rows of whole float4s and one part: a thread keeps its pieces between the two passes (up to 8,192 elements)
+template <int V>
+__global__ __launch_bounds__(256) void norm_rows4_k(const float* __restrict__ x, const float* __restrict__ w, float eps, int nd,
+                                                    float* __restrict__ out32, uint16_t* __restrict__ out16) {
+    __shared__ float red[4];
+    const int tid = threadIdx.x, n4 = nd >> 2;
+    const int64_t row = blockIdx.x;
+    const float4* xr = (const float4*)(x + row * nd);
+    float4 v[V];
+    float ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < V; i++) {
+        const int at = tid + i * 256;
+        v[i] = at < n4 ? xr[at] : make_float4(0.f, 0.f, 0.f, 0.f);
+        ss = fmaf(v[i].x, v[i].x, fmaf(v[i].y, v[i].y, fmaf(v[i].z, v[i].z, fmaf(v[i].w, v[i].w, ss))));
+    }
+    ss = block_sum(ss, red);
+    const float rinv = 1.0f / sqrtf(ss / (float)nd + eps);
+#pragma unroll
+    for (int i = 0; i < V; i++) {
+        const int at = tid + i * 256;
+        if (at >= n4) continue;
+        const float4 ww = ((const float4*)w)[at];
+        const float4 r = make_float4(v[i].x * rinv * ww.x, v[i].y * rinv * ww.y, v[i].z * rinv * ww.z, v[i].w * rinv * ww.w);
+        if (out32) ((float4*)(out32 + row * nd))[at] = r;
+        if (out16)
+            ((uint2*)(out16 + row * nd))[at] = make_uint2(to_bf16(r.x) | ((uint32_t)to_bf16(r.y) << 16), to_bf16(r.z) | ((uint32_t)to_bf16(r.w) << 16));
+    }
+}
+
+__global__ void group_scatter_k(GroupMat m, const float* __restrict__ rows, int64_t n) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    group_store(m, (int)(i / m.n_out), (int)(i % m.n_out), rows[i]);
+}
+
+__global__ void scaled_residual_k(float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ sa,
+                                  const float* __restrict__ b, const float* __restrict__ sb, int nd, int64_t n) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    const int j = (int)(i % nd);
+    float v = sa ? a[i] * sa[j] : a[i];
+    if (b) v += sb ? b[i] * sb[j] : b[i];
+    x[i] += v;
+}
+
+__global__ void add_rows_k(float* __restrict__ x, const float* __restrict__ rows, const float* __restrict__ vec, int nd, int64_t n) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    float v = x[i];
+    if (rows) v += rows[i];
+    if (vec) v += vec[i % nd];
+    x[i] = v;
+}
+
+__global__ void gather_rows_k(const float* __restrict__ src, const int32_t* __restrict__ idx, int nd, float* __restrict__ out, int64_t n) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    out[i] = src[(int64_t)idx[i / nd] * nd + i % nd];
+}
+
+bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
+
+Groups groups_of(const GroupP& p, int rows_per_group) {
+    Groups g{};
+    for (int i = 0; i < p.n_mats; i++) {
+        const int per = p.m[i].up ? (rows_per_group > 1 ? rows_per_group / 2 : 1) : rows_per_group;
+        g.first[i + 1] = g.first[i] + (p.m[i].n_out + per - 1) / per;
+    }
+    g.n = g.first[p.n_mats];
+    return g;
+}
+bool group_aligned(const GroupP& p) {
+    bool al = p.n_in % 8 == 0;
+    for (int i = 0; i < p.n_mats; i++) al = al && aligned16(p.m[i].w) && aligned16(p.m[i].up);
+    return al;
+}
+bool res_aligned(const ResP& p) {
+    bool al = true;
+    for (int i = 0; i < p.n_terms; i++) al = al && p.t[i].n_in % 8 == 0 && aligned16(p.t[i].w);
+    return al;
+}
+size_t padded(int n) { return (size_t)((n + CH - 1) / CH * CH); }
+constexpr size_t LDS_MAX = 144 * 1024;
+
+template <class F> bool allow_lds(F* fn, size_t lds) {
+    if (lds <= 64 * 1024) return true;
+    if (hipFuncSetAttribute((const void*)fn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS_MAX) == hipSuccess) return true;
+    (void)hipGetLastError();
+    return false;
+}
+
+template <int FMT, bool AL> bool launch_group(const GroupP& p, hipStream_t s) {
+    const size_t lds = padded(p.n_in) * sizeof(float);
+    Groups g4 = groups_of(p, 4);
+    if (g4.n >= 2048) {   // enough groups of four rows to keep every wave of the chip at work
+        if (!allow_lds(group_gemv_k<FMT, AL, 4>, lds)) return false;
+        hipLaunchKernelGGL((group_gemv_k<FMT, AL, 4>), dim3(min((g4.n + 3) / 4, 1024)), dim3(256), lds, s, p, g4);
+    } else {
+        Groups g2 = groups_of(p, 2);
+        if (!allow_lds(group_gemv_k<FMT, AL, 2>, lds)) return false;
+        hipLaunchKernelGGL((group_gemv_k<FMT, AL, 2>), dim3(min((g2.n + 3) / 4, 1024)), dim3(256), lds, s, p, g2);
+    }
+    return true;
+}
+template <int FMT, bool AL> bool launch_res(const ResP& p, hipStream_t s) {
+    size_t lds = 0;
+    for (int i = 0; i < p.n_terms; i++) lds += padded(p.t[i].n_in) * sizeof(float);
+    if (p.n_out >= 8192) {
+        if (!allow_lds(res_gemv_k<FMT, AL, 2>, lds)) return false;
+        hipLaunchKernelGGL((res_gemv_k<FMT, AL, 2>), dim3((p.n_out + 7) / 8), dim3(256), lds, s, p);
+    } else {
+        if (!allow_lds(res_gemv_k<FMT, AL, 1>, lds)) return false;
+        hipLaunchKernelGGL((res_gemv_k<FMT, AL, 1>), dim3((p.n_out + 3) / 4), dim3(256), lds, s, p);
+    }
+    return true;
+}
+
+// one call per (format, alignment)
+#define IT_BY_FORMAT(fmt, al, CALL)                                                    \
+    do {                                                                               \
+        if ((fmt) == W_BF16) { if (al) { CALL(W_BF16, true); } else { CALL(W_BF16, false); } } \
+        else if ((fmt) == W_F16) { if (al) { CALL(W_F16, true); } else { CALL(W_F16, false); } } \
+        else { if (al) { CALL(W_F32, true); } else { CALL(W_F32, false); } }           \
+    } while (0)
+
+}  // namespace
+
+bool group_gemv_takes(const GroupP& p) { return p.n_tok == 1 && padded(p.n_in) * sizeof(float) <= LDS_MAX; }
+bool group_gemv(const GroupP& p, hipStream_t s) {
+    if (!group_gemv_takes(p)) return false;
+    const bool al = group_aligned(p);
+    bool ok = false;
+#define IT_CALL(F, A) ok = launch_group<F, A>(p, s)
+    IT_BY_FORMAT(p.fmt, al, IT_CALL);
+#undef IT_CALL
+    return ok;
+}
+
+bool res_gemv_takes(const ResP& p) {
+    size_t lds = 0;
+    for (int i = 0; i < p.n_terms; i++) lds += padded(p.t[i].n_in) * sizeof(float);
+    return p.n_tok == 1 && lds <= LDS_MAX;
+}
+bool res_gemv(const ResP& p, hipStream_t s) {
+    if (!res_gemv_takes(p)) return false;
+    const bool al = res_aligned(p);
+    bool ok = false;
+#define IT_CALL(F, A) ok = launch_res<F, A>(p, s)
+    IT_BY_FORMAT(p.fmt, al, IT_CALL);
+#undef IT_CALL
+    return ok;
+}
+
+void group_rows(const GroupP& p, hipStream_t s) {
+    const Groups g = groups_of(p, 1);
+    const bool al = group_aligned(p);
+    const dim3 grid((g.n + 3) / 4, (p.n_tok + NT - 1) / NT);
+#define IT_CALL(F, A) hipLaunchKernelGGL((group_rows_k<F, A>), grid, dim3(256), 0, s, p, g)
+    IT_BY_FORMAT(p.fmt, al, IT_CALL);
+#undef IT_CALL
+}
+void res_rows(const ResP& p, hipStream_t s) {
+    const bool al = res_aligned(p);
+    const dim3 grid((p.n_out + 3) / 4, (p.n_tok + NT - 1) / NT);
+#define IT_CALL(F, A) hipLaunchKernelGGL((res_rows_k<F, A>), grid, dim3(256), 0, s, p)
+    IT_BY_FORMAT(p.fmt, al, IT_CALL);
+#undef IT_CALL
+}
+
+void norm_rows(const float* x, const float* w, int groups, float eps, int64_t n_rows, int nd, float* out32, uint16_t* out16, hipStream_t s) {
+    if (n_rows <= 0) return;
+    if (w && groups == 1 && nd % 8 == 0 && nd <= 8192 && aligned16(x) && aligned16(w) && aligned16(out32) && aligned16(out16)) {
+        if (nd <= 1024) hipLaunchKernelGGL(norm_rows4_k<1>, dim3((unsigned)n_rows), dim3(256), 0, s, x, w, eps, nd, out32, out16);
+        else if (nd <= 2048) hipLaunchKernelGGL(norm_rows4_k<2>, dim3((unsigned)n_rows), dim3(256), 0, s, x, w, eps, nd, out32, out16);
+        else if (nd <= 4096) hipLaunchKernelGGL(norm_rows4_k<4>, dim3((unsigned)n_rows), dim3(256), 0, s, x, w, eps, nd, out32, out16);
+        else hipLaunchKernelGGL(norm_rows4_k<8>, dim3((unsigned)n_rows), dim3(256), 0, s, x, w, eps, nd, out32, out16);
+        return;
+    }
+    hipLaunchKernelGGL(norm_rows_k, dim3((unsigned)n_rows, groups), dim3(256), 0, s, x, w, groups, eps, nd, out32, out16);
+}
+
+static dim3 per_element(int64_t n) { return dim3((unsigned)((n + 255) / 256)); }
+void group_scatter(const GroupMat& m, const float* rows, int n_tok, hipStream_t s) {
+    const int64_t n = (int64_t)n_tok * m.n_out;
+    hipLaunchKernelGGL(group_scatter_k, per_element(n), dim3(256), 0, s, m, rows, n);
+}
+void scaled_residual(float* x, const float* a, const float* sa, const float* b, const float* sb, int64_t n_rows, int nd, hipStream_t s) {
+    const int64_t n = n_rows * nd;
+    hipLaunchKernelGGL(scaled_residual_k, per_element(n), dim3(256), 0, s, x, a, sa, b, sb, nd, n);
+}
+void add_rows(float* x, const float* rows, const float* vec, int64_t n_rows, int nd, hipStream_t s) {
+    const int64_t n = n_rows * nd;
+    hipLaunchKernelGGL(add_rows_k, per_element(n), dim3(256), 0, s, x, rows, vec, nd, n);
+}
+void gather_rows(const float* src, const int32_t* idx, int n_rows, int nd, float* out, hipStream_t s) {
+    const int64_t n = (int64_t)n_rows * nd;
+    hipLaunchKernelGGL(gather_rows_k, per_element(n), dim3(256), 0, s, src, idx, nd, out, n);
+}
+
+}  // namespace itk

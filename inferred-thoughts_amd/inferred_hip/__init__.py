@@ -14,7 +14,7 @@ from pathlib import Path
 import numpy as np
 
 F32, F16, Q8_0, BF16, NVFP4 = 0, 1, 8, 30, 40
-EXACT, NO_GRAPH, NO_FUSE, NO_CHAIN = 1, 2, 4, 8
+EXACT, NO_GRAPH, NO_FUSE, NO_CHAIN, F32_MODE = 1, 2, 4, 8, 16
 
 _HERE = Path(__file__).resolve().parent
 # INFERRED_HIP_LIB names another build of the library (comparing two builds on one machine)
@@ -47,6 +47,28 @@ class Delta(C.Structure):
                 ("beta", C.c_void_p), ("ssm_a", C.c_void_p), ("dt_bias", C.c_void_p),
                 ("n_tokens", c_u64), ("head_k_dim", c_u64), ("head_v_dim", c_u64),
                 ("n_k_heads", c_u64), ("n_v_heads", c_u64)]
+
+
+class GroupMat(C.Structure):
+    _fields_ = [("w", Weights), ("up", Weights), ("out", C.c_void_p), ("out_len", c_u64), ("slab", C.c_void_p),
+                ("slab_len", c_u64), ("slab_row", c_u64), ("head_dim", c_u64), ("head_stride", c_u64), ("scale", c_f32),
+                ("_pad", c_u32)]
+
+
+class ResTerm(C.Structure):
+    _fields_ = [("w", Weights), ("inp", C.c_void_p), ("in_len", c_u64), ("scale", C.c_void_p), ("norm_w", C.c_void_p),
+                ("norm_groups", c_u64), ("eps", c_f32), ("_pad", c_u32)]
+
+
+class AttnBias(C.Structure):
+    _fields_ = [("q", C.c_void_p), ("q_len", c_u64), ("k", C.c_void_p), ("v", C.c_void_p), ("k_len", c_u64), ("v_len", c_u64)] + \
+               [(n, c_u64) for n in ("n_pos", "k_dim", "v_dim", "k_stride", "v_stride", "n_head", "n_head_kv")] + \
+               [("scale", c_f32), ("sink", c_u32), ("slopes", C.c_void_p), ("temp_coef", c_f32), ("temp_every", c_u32)]
+
+
+class Mamba2(C.Structure):
+    _fields_ = [(n, C.c_void_p) for n in ("conv_w", "conv_b", "dt_bias", "a_log", "d")] + \
+               [(n, c_u64) for n in ("heads", "vdim", "n", "groups", "taps", "pos")]
 
 
 class Route(C.Structure):
@@ -102,7 +124,9 @@ it_engine_decode_greedy it_engine_last_error it_engine_ssm_state it_engine_conv_
 it_engine_v_slab it_synth_write_gguf it_hip_attend_noalloc it_hip_reserve_for_weights it_hip_reserve_for_kv
 it_hip_set_prefetch it_hip_set_model_path it_hip_set_map_base it_hip_expert_coverage it_hip_replace_experts_by_counts
 it_hip_expert_counts it_hip_mean_streams it_hip_mul_rows it_hip_silu it_hip_sigmoid it_hip_mul_streams it_hip_row_dot
-it_hip_signed_sqrt_sigmoid it_hip_dilated_conv it_hip_qsa_pool it_hip_qsa_select it_hip_attend_sparse""".split()
+it_hip_signed_sqrt_sigmoid it_hip_dilated_conv it_hip_qsa_pool it_hip_qsa_select it_hip_attend_sparse
+it_hip_norm_matmuls it_hip_matmul_residual it_hip_attend_bias it_hip_mamba2 it_hip_add_rows it_hip_gather_rows it_hip_is_f32
+it_hip_zero_slab it_engine_forward_rows""".split()
 
 _lib = None
 
@@ -224,6 +248,15 @@ def lib() -> C.CDLL:
         "it_engine_restore": (C.c_int, [vp, u64, vp, vp]),
         "it_engine_rewind": (C.c_int, [vp, u64]),
         "it_engine_forward": (C.c_int, [vp, vp, u64, vp]),
+        "it_engine_forward_rows": (C.c_int, [vp, vp, u64, vp, u64, vp]),
+        "it_hip_norm_matmuls": (None, [vp, vp, u64, vp, u64, f32, vp, u64]),
+        "it_hip_matmul_residual": (None, [vp, vp, u64, vp, u64]),
+        "it_hip_attend_bias": (None, [vp, vp, vp, u64]),
+        "it_hip_mamba2": (None, [vp, vp, vp, u64, vp, u64, vp, u64, vp, u64]),
+        "it_hip_add_rows": (None, [vp, vp, u64, vp, vp, u64]),
+        "it_hip_gather_rows": (None, [vp, vp, u64, u64, vp, u64, vp, u64]),
+        "it_hip_is_f32": (C.c_int, [vp]),
+        "it_hip_zero_slab": (None, [vp, vp]),
         "it_engine_prefill": (C.c_int, [vp, vp, u64, vp]),
         "it_engine_generate": (C.c_int64, [vp, vp, u64, u64, vp, vp]),
         "it_engine_decode_greedy": (C.c_int64, [vp, u64, vp]),
@@ -281,14 +314,15 @@ def attend_noalloc(q_ptr: int, q_len: int, k_ptr: int, v_ptr: int, kv_len: int, 
 class Hip:
     """One backend instance: `Cuda::new` of the reference, for gfx950."""
 
-    def __init__(self, exact: bool = False, graph: bool = True, device: int = 0, fuse: bool = True, chain: bool = True):
+    def __init__(self, exact: bool = False, graph: bool = True, device: int = 0, fuse: bool = True, chain: bool = True,
+                 f32: bool = False):
         self.L = lib()
         err = C.create_string_buffer(512)
-        flags = (EXACT if exact else 0) | (0 if graph else NO_GRAPH) | (0 if fuse else NO_FUSE) | (0 if chain else NO_CHAIN)
+        flags = (EXACT if exact else 0) | (0 if graph else NO_GRAPH) | (0 if fuse else NO_FUSE) | (0 if chain else NO_CHAIN) | (F32_MODE if f32 else 0)
         self.h = self.L.it_hip_create(flags, device, err, 512)
         if not self.h:
             raise HipError(err.value.decode())
-        self.exact = exact
+        self.exact, self.f32 = exact, f32 or exact
 
     def close(self):
         if self.h:
@@ -398,6 +432,28 @@ class Hip:
     def moe_finish(self, out, at, n, rows, route: Route, shared, logit, logit_at):
         self.L.it_hip_moe_finish(self.h, _p(out), out.size, at, n, _p(rows), rows.size, C.addressof(route),
                                  _p(shared), shared.size, _p(logit), logit.size, logit_at)
+
+    # ---- ops of models with unquantized matrices ----
+    def norm_matmuls(self, x, norm_w, n_in, eps, mats: list[GroupMat]):
+        a = (GroupMat * len(mats))(*mats)
+        self.L.it_hip_norm_matmuls(self.h, _p(x), x.size, _p(norm_w), n_in, eps, a, len(mats))
+
+    def matmul_residual(self, x, terms: list[ResTerm]):
+        a = (ResTerm * len(terms))(*terms)
+        self.L.it_hip_matmul_residual(self.h, _p(x), x.size, a, len(terms))
+
+    def attend_bias(self, a: AttnBias, out):
+        self.L.it_hip_attend_bias(self.h, C.addressof(a), _p(out), out.size)
+
+    def mamba2(self, m: Mamba2, u, ring, state, out):
+        self.L.it_hip_mamba2(self.h, C.addressof(m), _p(u), u.size, _p(ring), ring.size, _p(state), state.size, _p(out), out.size)
+
+    def add_rows(self, x, rows, vec):
+        self.L.it_hip_add_rows(self.h, _p(x), x.size, _p(rows), _p(vec), vec.size)
+
+    def gather_rows(self, src, width, idx, out):
+        i = np.ascontiguousarray(idx, np.uint32)
+        self.L.it_hip_gather_rows(self.h, _p(src), src.size, width, _p(i), i.size, _p(out), out.size)
 
     # ---- residency ----
     def host_wrote(self, buf):
@@ -622,6 +678,15 @@ class Engine:
         if rc:
             self._err(rc)
         return logits
+
+    def forward_rows(self, tokens, rows):
+        """Passes over `tokens` in batches of max_batch; the logits [len(rows), n_vocab] of the tokens `rows`."""
+        t, r = np.ascontiguousarray(tokens, dtype=np.uint32), np.ascontiguousarray(rows, dtype=np.uint32)
+        out = np.empty((r.size, self.model.n_vocab), np.float32)
+        rc = self.L.it_engine_forward_rows(self.h, _p(t), t.size, _p(r), r.size, _p(out))
+        if rc:
+            self._err(rc)
+        return out
 
     def prefill(self, tokens, want_logits=True):
         t = np.ascontiguousarray(tokens, dtype=np.uint32)
