@@ -263,6 +263,7 @@ it_hip::Act* it_hip::act_slot(const float* host, size_t len) {
 float* it_hip::act_in(const float* host, size_t len) {
     Act* a = act_slot(host, len);
     if (!a) return nullptr;
+    if (a->dev_current && a->elided && a->h_valid) act_widen(*a);
     if (a->dev_current && a->elided) {
         fail("an op reads a buffer whose producer was folded into a fused kernel that does not write it");
         return nullptr;
@@ -2065,6 +2066,7 @@ void it_hip_host_needs(it_hip* be, float* buf, uint64_t len) {
     auto it = be->acts.find(buf);
     if (it == be->acts.end() || !it->second.dev_current) return;
     if (!be->held.empty()) be->release_held();
+    if (it->second.elided && it->second.h_valid) be->act_widen(it->second);
     if (it->second.elided) {
         be->fail("host_needs: the op that writes this buffer was folded into a fused kernel that does not write it");
         return;

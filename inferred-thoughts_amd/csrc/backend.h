@@ -93,6 +93,7 @@ struct it_hip {
     uint16_t* act_half_out(const float* host, size_t rows, size_t row);
     uint16_t* act_half_reserve(Act& a, size_t rows, size_t row);
     const uint16_t* act_half_if_valid(const float* host, size_t rows, size_t row);
+    void act_widen(Act& a);                  // the f32 mirror of rows that exist in bf16 only
     // scratch of the unquantized ops, by use: f32 rows, bf16 rows
     struct Tmp { void* p = nullptr; size_t bytes = 0; };
     Tmp tmps[6];

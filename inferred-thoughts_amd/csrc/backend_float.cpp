@@ -74,6 +74,11 @@ uint16_t* it_hip::act_half_out(const float* host, size_t rows, size_t row) {
     a->h_valid = true;
     return h;
 }
+void it_hip::act_widen(Act& a) {
+    if (a.cap < a.h_rows * a.h_row) return;
+    widen_rows(a.h16, (int64_t)a.h_rows, (int)a.h_row, a.dev, stream);
+    if (check(hipGetLastError(), "kernel launch")) a.elided = false;
+}
 const uint16_t* it_hip::act_half_if_valid(const float* host, size_t rows, size_t row) {
     auto it = acts.find(host);
     if (it == acts.end() || !it->second.h_valid || !it->second.dev_current || it->second.h_rows != rows || it->second.h_row != row) return nullptr;
@@ -408,7 +413,7 @@ void it_hip_mamba2(it_hip* be, const it_mamba2* m, const float* u, uint64_t u_le
     p.heads = (int)m->heads; p.vdim = (int)m->vdim; p.n = (int)m->n; p.groups = (int)m->groups; p.taps = (int)m->taps;
     p.n_tok = (int)n;
     p.pos = (int)m->pos;
-    REQUIRE(ssd_takes(p), "mamba2: a state of at most 256 columns and at most 16 taps");
+    REQUIRE(ssd_takes(p), "mamba2: a state of at most 512 columns and at most 16 taps");
     p.accurate = be->f32 || !be->fuse_enabled;
     p.u = be->act_in(u, u_len);
     p.conv_w = be->const_in(m->conv_w, ch * m->taps);

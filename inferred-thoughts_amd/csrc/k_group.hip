@@ -364,6 +364,11 @@ __global__ __launch_bounds__(256) void norm_rows4_k(const float* __restrict__ x,
     }
 }
 
+__global__ void widen_rows_k(const uint16_t* __restrict__ in, int nd, float* __restrict__ out, int64_t n) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i < n) out[i] = it_bf16_to_f32(in[i / nd * pad8(nd) + i % nd]);
+}
+
 __global__ void group_scatter_k(GroupMat m, const float* __restrict__ rows, int64_t n) {
     const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (i >= n) return;
@@ -517,6 +522,10 @@ void norm_rows(const float* x, const float* w, int groups, float eps, int64_t n_
 }
 
 static dim3 per_element(int64_t n) { return dim3((unsigned)((n + 255) / 256)); }
+void widen_rows(const uint16_t* in, int64_t n_rows, int nd, float* out, hipStream_t s) {
+    const int64_t n = n_rows * nd;
+    hipLaunchKernelGGL(widen_rows_k, per_element(n), dim3(256), 0, s, in, nd, out, n);
+}
 void group_scatter(const GroupMat& m, const float* rows, int n_tok, hipStream_t s) {
     const int64_t n = (int64_t)n_tok * m.n_out;
     hipLaunchKernelGGL(group_scatter_k, per_element(n), dim3(256), 0, s, m, rows, n);

@@ -25,7 +25,7 @@ namespace {
 typedef float v4f __attribute__((ext_vector_type(4)));
 constexpr int PR = 16;     // value rows per block
 constexpr int TAPS_MAX = 16;
-constexpr int N_MAX = 256;
+constexpr int N_MAX = 512;
 
 IT_DEV float silu_of(float z, int accurate) { return accurate ? silu_exact(z) : fx_silu(z); }
 
@@ -365,7 +365,8 @@ template <class F> bool allow_lds(F* fn, size_t lds) {
         else if ((n) <= 32) { CALL(2); }    \
         else if ((n) <= 64) { CALL(4); }    \
         else if ((n) <= 128) { CALL(8); }   \
-        else { CALL(16); }                  \
+        else if ((n) <= 256) { CALL(16); }  \
+        else { CALL(32); }                  \
     } while (0)
 
 unsigned blocks(const SsdP& p) { return (unsigned)(p.heads * ((p.vdim + PR - 1) / PR)); }

@@ -72,6 +72,8 @@ void res_gemm_bf16(const ResP& p, const uint16_t* const in16[RES_MAX], hipStream
 // to f32 and / or to bf16 rows of pad8(nd)
 void norm_rows(const float* x, const float* w, int groups, float eps, int64_t n_rows, int nd, float* out32, uint16_t* out16,
                hipStream_t s);
+// f32 rows of nd from bf16 rows of pad8(nd)
+void widen_rows(const uint16_t* in, int64_t n_rows, int nd, float* out, hipStream_t s);
 // one matrix's f32 rows to where its GroupOut says (the form with one launch per operation)
 void group_scatter(const GroupMat& m, const float* rows, int n_tok, hipStream_t s);
 // x += a * sa (+ b * sb), the sum of the two first; scales [nd] or null, b may be null

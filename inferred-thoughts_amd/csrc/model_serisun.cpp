@@ -120,7 +120,7 @@ struct Serisun : it_model {
                     return false;
                 if (m.heads % m.groups) return fail("config.json: " + wm + ": heads do not divide into groups");
                 if (m.inner() % m.norm_groups) return fail("config.json: " + wm + ": the inner width does not divide into norm_groups");
-                if (m.state > 256 || m.taps > 16) return fail("config.json: " + wm + ": a state of more than 256 columns or more than 16 taps");
+                if (m.state > 512 || m.taps > 16) return fail("config.json: " + wm + ": a state of more than 512 columns or more than 16 taps");
             } else {
                 return fail("config.json: " + where + ": unknown mixer '" + ty->str + "'");
             }

@@ -1,0 +1,319 @@
+"""Serisun models through the framework's engine against the plain oracle: prefill, decoding through the cache, portions,
+used-again caches, several requests at once, recorded graphs, greedy generation, and the trace runner."""
+import json
+import os
+import subprocess
+import sys
+from pathlib import Path
+
+import numpy as np
+import pytest
+
+import serisun_ref as ref
+from serisun_util import CONFIGS, attention, config, logit_error, mamba2, weights, write
+
+pytestmark = pytest.mark.gpu
+ROOT = Path(__file__).resolve().parent.parent
+MODES = {"bf16": {}, "f32": {"f32": True}, "steps": {"fuse": False}}
+LIMIT = {"bf16": 2e-2, "f32": 1e-4, "steps": 2e-2}
+
+
+class Case:
+    def __init__(self, folder, cfg, seed=0, w=None):
+        import inferred_hip as ih
+        self.cfg, self.w = cfg, w if w is not None else weights(cfg, seed)
+        self.path = write(folder, cfg, self.w)
+        self.model = ih.Model(self.path)
+        self.cache = {}
+
+    def logits(self, tokens):
+        key = tuple(int(t) for t in tokens)
+        if key not in self.cache:
+            self.cache[key] = ref.forward(tokens, self.cfg, self.w)
+        return self.cache[key]
+
+    def tokens(self, n, seed=0):
+        return np.random.default_rng(seed).integers(0, self.cfg["vocab"], n)
+
+
+@pytest.fixture(scope="module")
+def cases(tmp_path_factory):
+    return {k: Case(tmp_path_factory.mktemp("serisun") / k, c, i) for i, (k, c) in enumerate(CONFIGS.items())}
+
+
+@pytest.fixture(params=sorted(MODES))
+def be(request):
+    import inferred_hip as ih
+    b = ih.Hip(**MODES[request.param])
+    b.name, b.limit = request.param, LIMIT[request.param]
+    yield b
+    err = b.take_error()
+    b.close()
+    assert err is None, err
+
+
+def engine(case, be, n_ctx, max_batch=512):
+    import inferred_hip as ih
+    return ih.Engine(case.model, be, n_ctx, max_batch)
+
+
+def feed(e, tokens, sizes):
+    """The logits of every token, fed in portions of the given sizes (the last one repeated)."""
+    out, at, k = [], 0, 0
+    while at < len(tokens):
+        c = min(sizes[min(k, len(sizes) - 1)], len(tokens) - at)
+        out.append(e.forward_rows(tokens[at:at + c], np.arange(c)))
+        at, k = at + c, k + 1
+    return np.concatenate(out)
+
+
+def held(got, want, be, what=""):
+    e = logit_error(got, want)
+    assert np.isfinite(got).all()
+    # (a norm over three channels that are all near zero multiplies a 16-bit rounding: one token in fifty may be up to four times as far)
+    assert (e > be.limit).sum() <= (max(1, len(e) // 50) if be.limit > 1e-3 else 0) and e.max() < 4 * be.limit, f"{what}: {e.max():.2e} at token {int(e.argmax())}"
+
+
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+@pytest.mark.parametrize("n", [1, 2, 7, 16, 17, 64, 65, 129, 200])
+def test_a_whole_prompt(cases, be, name, n):
+    c, e = cases[name], None
+    e = engine(c, be, n)
+    t = c.tokens(n)
+    held(feed(e, t, [n]), c.logits(t), be)
+    e.close()
+
+
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_residual_stream_after_every_layer_run(cases, be, name):
+    """Layer by layer: the first run that differs is the faulty one."""
+    c = cases[name]
+    t = c.tokens(30, 4)
+    want = []
+    ref.forward(t, c.cfg, c.w, want)
+    for n in (30, 1):
+        got = []
+        e = engine(c, be, 40)
+        e.set_trace(lambda what, run, v: got.append((run, v.reshape(n, -1))) if what == "post_layer" else None)
+        e.forward(t[:n])
+        e.close()
+        assert [r for r, _ in got] == list(range(len(want)))
+        for (run, v), w in zip(got, want):
+            d = np.sqrt(((v - w[:n]) ** 2).mean() / (w[:n] ** 2).mean())
+            assert d < be.limit, f"run {run}: {d:.2e}"
+
+
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+@pytest.mark.parametrize("sizes", [[1], [2], [3, 2, 2, 11], [16, 1, 17, 64, 2], [63, 2, 1], [64, 64, 1], [65, 2], [150, 1]])
+def test_portions_of_any_size(cases, be, name, sizes):
+    """The logits at a position do not depend on how the prompt was cut: single tokens, pairs, and cuts just before, at and
+    just after a tile's and a chunk's edge."""
+    c = cases[name]
+    t = c.tokens(170, 1)
+    e = engine(c, be, 170)
+    held(feed(e, t, sizes), c.logits(t), be, str(sizes))
+    e.close()
+
+
+def test_a_prompt_longer_than_the_engine_batch(cases, be):
+    c = cases["mixed"]
+    t = c.tokens(100, 2)
+    e = engine(c, be, 128, max_batch=24)
+    held(feed(e, t, [100]), c.logits(t), be)
+    assert e.pos == 100
+    e.reset()
+    held(e.prefill(t)[None], c.logits(t)[-1:], be)
+    e.close()
+
+
+@pytest.mark.parametrize("name", ["mixed", "odd"])
+def test_a_cache_that_is_used_again(cases, be, name):
+    """Requests of unequal lengths one after the other on one engine: nothing of the last one is left."""
+    c = cases[name]
+    e = engine(c, be, 150)
+    for k, n in enumerate((150, 3, 80, 1, 40)):
+        t = c.tokens(n, 10 + k)
+        e.reset()
+        held(feed(e, t, [max(1, n // 2), 1, 2]), c.logits(t), be, f"request {k}")
+    e.close()
+
+
+def test_requests_that_take_turns(cases, be):
+    """Three requests of unequal lengths on engines of their own over one backend, portions interleaved; one ends and its
+    engine serves another meanwhile."""
+    c = cases["mixed"]
+    es = [engine(c, be, 90) for _ in range(3)]
+    ts = [c.tokens(n, 20 + n) for n in (90, 31, 64)]
+    at, got = [0, 0, 0], [[], [], []]
+    r = np.random.default_rng(0)
+    again = False
+    while any(a < len(t) for a, t in zip(at, ts)):
+        for k in range(3):
+            n = min(int(r.choice([1, 1, 2, 5, 20])), len(ts[k]) - at[k])
+            if n:
+                got[k].append(es[k].forward_rows(ts[k][at[k]:at[k] + n], np.arange(n)))
+                at[k] += n
+        if at[1] == len(ts[1]) and not again:
+            again = True
+            held(np.concatenate(got[1]), c.logits(ts[1]), be)
+            es[1].reset()
+            ts[1], at[1], got[1] = c.tokens(50, 99), 0, []
+    for k in range(3):
+        held(np.concatenate(got[k]), c.logits(ts[k]), be, f"request {k}")
+    for e in es:
+        e.close()
+
+
+@pytest.mark.parametrize("name", ["mixed", "wide", "all_looped", "odd"])
+def test_long_decoding_from_recorded_graphs(cases, name):
+    """Hundreds of single-token passes, most of them replays of one recorded graph, checked against the whole sequence; eager
+    work (a portion, a checkpoint) in between; every pass equal to the eager backend's."""
+    import inferred_hip as ih
+    c = cases[name]
+    t = c.tokens(330, 3)
+    want = c.logits(t)
+    runs = {}
+    for graph in (True, False):
+        b = ih.Hip(graph=graph)
+        e = engine(c, b, 330)
+        got = [feed(e, t[:20], [20])]
+        for p in range(20, 330):
+            if p in (150, 151):
+                e.checkpoint()
+            if p in (200, 201, 202):
+                continue
+            if p == 203:
+                got.append(e.forward_rows(t[200:204], np.arange(4)))
+                continue
+            got.append(e.forward_rows(t[p:p + 1], [0]))
+        runs[graph] = np.concatenate(got)
+        s = b.graph_stats()
+        assert b.take_error() is None
+        assert (s["replays"] > 250 and s["captures"] >= 1) if graph else s["captures"] == 0
+        e.close()
+        b.close()
+        assert logit_error(runs[graph], want).max() < 2e-2
+    assert np.array_equal(runs[True], runs[False])
+
+
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_greedy_generation(cases, name):
+    """The framework's own generation, with ids chosen on the host (generate) and fed back on the device (decode_greedy), against
+    the oracle's arg-max, token by token as long as its choice is clear."""
+    import inferred_hip as ih
+    c = cases[name]
+    t = [int(x) for x in c.tokens(23, 7)]
+    for kw in (dict(f32=True), {}):
+        b = ih.Hip(**kw)
+        e = engine(c, b, 80, max_batch=16)
+        ids, _ = e.generate(t, 40)
+        e.reset()
+        e.prefill(t)
+        dev = e.decode_greedy(40)
+        e.close()
+        assert b.take_error() is None
+        b.close()
+        assert len(ids) == 40 and list(ids) == list(dev)
+        seq = list(t)
+        lim = 1e-4 if kw else 2e-2
+        for i in ids:
+            y = ref.forward(seq, c.cfg, c.w)[-1]
+            top = np.sort(y)[-2:]
+            if top[1] - top[0] < 8 * lim * y.std():
+                break
+            assert int(i) == int(y.argmax())
+            seq.append(int(i))
+        assert len(seq) > len(t) + (10 if kw else 0)
+
+
+def test_checkpoint_and_restore(cases, be):
+    c = cases["mixed"]
+    t = c.tokens(60, 8)
+    e = engine(c, be, 60)
+    feed(e, t[:25], [25])
+    ck = e.checkpoint()
+    first = feed(e, t[25:], [9, 1, 2])
+    e.restore(ck)
+    assert e.pos == 25 and not e.rewind(3)
+    again = feed(e, t[25:], [9, 1, 2])
+    assert np.array_equal(first, again)
+    held(again, c.logits(t)[25:], be)
+    e.close()
+
+
+def test_other_tensor_types_and_errors(cases, be, tmp_path):
+    """Matrices in f32 and f16 beside bf16 ones; tokens and positions that are refused."""
+    import inferred_hip as ih
+    cfg = CONFIGS["odd"]
+    w = weights(cfg, 3)
+    c = Case(tmp_path / "m", cfg, w=w)
+    d = write(tmp_path / "n", cfg, w, {"l1.mix.q": "F32", "l0.mix.in": "F16", "embed": "F32", "head": "F16", "l2.mlp.down": "F32", "l3.norm1": "F16"})
+    m = ih.Model(d)
+    t = c.tokens(70, 1)
+    e = ih.Engine(m, be, 70)
+    held(feed(e, t, [40, 1, 3, 20]), c.logits(t), be)
+    with pytest.raises(ih.HipError, match="context overflow"):
+        e.forward([1])
+    e.reset()
+    with pytest.raises(ih.HipError, match="outside the vocabulary"):
+        e.forward([cfg["vocab"]])
+    with pytest.raises(ih.HipError, match="ascend"):
+        e.forward_rows([1, 2, 3], [2, 1])
+    e.close()
+    m.close()
+
+
+def test_a_key_far_back_decides_the_logits(tmp_path, be):
+    """Planted weights: one token's key answers one token's query from anywhere in the sequence.  The answer's logits carry the
+    planted token's value, from every distance (tile and split edges included), prefilled and decoded."""
+    cfg = config([attention(2, 1, 16, 16, temp=False, scale=1.0)], width=32, vocab=12, ff=None, logit_scale=1.0, eps=1e-6)
+    w = {k: np.zeros_like(v) for k, v in weights(cfg, 0).items()}
+    for k in ("l0.norm1", "l0.ls1", "final.norm"):
+        w[k][:] = 1.0
+    w["embed"][np.arange(12), np.arange(12)] = 1.0                   # a channel per token, after the norm about 5.7
+    for h in range(2):
+        w["l0.mix.q"][16 * h, 1] = 4.0                               # token 1 asks
+    w["l0.mix.k"][0, 2] = 4.0                                        # token 2 answers
+    w["l0.mix.v"][3, 2] = 1.0
+    w["l0.mix.o"][20, 3] = w["l0.mix.o"][20, 19] = 1.0
+    w["head"][5, 20] = w["head"][7, 1] = 1.0
+    c = Case(tmp_path / "m", cfg, w=w)
+    for far in (0, 1, 62, 63, 64, 65, 127, 128, 129, 200):
+        t = np.full(260, 4)
+        t[far], t[far + 1:] = 2, np.where(np.arange(259 - far) % 3 == 0, 1, 4)
+        want = c.logits(t)
+        assert want[-1 if t[-1] == 1 else -2 if t[-2] == 1 else -3, 5] > 1.0
+        e = engine(c, be, 260)
+        got = feed(e, t, [far + 2, 1, 1, 30, 1])
+        assert np.abs(got - want).max() < (3e-2 if be.name == "bf16" else 1e-2 if be.name == "steps" else 1e-4)
+        e.close()
+
+
+# ---------------------------------------------------------------- the trace runner
+@pytest.mark.parametrize("dtype", ["bfloat16", "float32"])
+def test_the_trace_runner(cases, tmp_path, dtype):
+    c = cases["mixed"]
+    reqs = {"a": c.tokens(50, 1), "b": c.tokens(3, 2), "c": c.tokens(20, 3)}
+    steps, at = [], {k: 0 for k in reqs}
+    for name, n in [("a", 30), ("a", 1), ("a", 19), ("b", 3), ("c", 2), ("c", 18)]:
+        lo = at[name]
+        at[name] += n
+        want = [] if (name, n) == ("c", 2) else [n - 1] if n < 3 else [2, 0, n - 1]   # in any order
+        steps.append({"step": len(steps), "entries": [{"id": name, "tokens": [int(x) for x in reqs[name][lo:lo + n]], "want": want}],
+                      "end": [name] if at[name] == len(reqs[name]) else []})
+    env = {k: v for k, v in os.environ.items() if k != "HOME"}
+    p = subprocess.run([str(ROOT / "bin" / "trace_run"), "--model", str(c.path), "--dtype", dtype, "--out", str(tmp_path), "--max-tokens", "50"],
+                       input="".join(json.dumps(s) + "\n" for s in steps), stdout=subprocess.PIPE, stderr=subprocess.PIPE, text=True, timeout=90, env=env)
+    assert p.returncode == 0, p.stderr[-2000:]
+    assert [x for x in p.stdout.splitlines() if x.startswith("done")] == [f"done {i}" for i in range(len(steps))]
+    lo = {k: 0 for k in reqs}
+    for s in steps:
+        x = s["entries"][0]
+        f = tmp_path / f"{s['step']}.f32"
+        if x["want"]:
+            got = np.fromfile(f, "<f4").reshape(len(x["want"]), c.cfg["vocab"])
+            want = c.logits(reqs[x["id"]])[[lo[x["id"]] + k for k in x["want"]]]
+            assert logit_error(got, want).max() < (1e-4 if dtype == "float32" else 2e-2)
+        else:
+            assert not f.exists()
+        lo[x["id"]] += len(x["tokens"])
