@@ -267,6 +267,9 @@ def main():
                          "is cold and fetched from the model file when a layer picks it (0 = no host tier)")
     ap.add_argument("--no-prefetch", action="store_true",
                     help="with a cold tier: do not read the next layer's likely experts ahead (set_prefetch off)")
+    ap.add_argument("--serisun", metavar="SIZES", nargs="?", const="w1024,w2048,w4096", default="",
+                    help="another run: prefill and decode of random-weight Serisun models of these sizes (comma-separated, default "
+                         "all) beside qwen35moe models of equal size, with both designs' kernels; prints its own JSON line")
     ap.add_argument("--summarize-profile", metavar="DIR",
                     help="no run: print the profiles/ summary of the rocprofv3 outputs under DIR (trace/, pmc_FETCH_SIZE/, "
                          "pmc_WRITE_SIZE/ of --decode-only runs) and exit")
@@ -284,6 +287,13 @@ def main():
         from inferred_hip import single_ops
         ffn = [int(t) for t in args.ffn_tokens.split(",") if t]
         print(json.dumps({"single_op": single_ops.run(ih, seed=args.seed, exact=args.exact, ffn_tokens=ffn)}), flush=True)
+        return
+    if args.serisun:
+        import tempfile
+        from inferred_hip import serisun_bench
+        with tempfile.TemporaryDirectory(dir=str(model_path(args).parent)) as d:
+            rows = serisun_bench.run(ih, Path(d), args.serisun.split(","), steps=args.steps, seed=args.seed)
+        print(json.dumps({"serisun": rows}), flush=True)
         return
     import torch
 

@@ -352,6 +352,8 @@ struct it_hip {
             return;
         }
         rec.run = f;
+        rec.fam = fam;
+        rec.bytes = bytes;
         pending.push_back(std::move(rec));
         pass_signature.push_back(sig);
         if (mode == Mode::Deferred) return;

@@ -1230,7 +1230,8 @@ void it_hip::run_fused(std::vector<OpRec>& ops) {
             n++;
         }
         if (!pl.consumed[i]) {
-            Span sp(this, FAM_OTHER, 0);
+            const bool whole_step = ops[i].id >= OP_GROUP && ops[i].id < OP_QUANT;   // an unquantized model's op is a fused step by itself
+            Span sp(this, whole_step ? ops[i].fam : FAM_OTHER, whole_step ? ops[i].bytes : 0);
             ops[i].run(stream);
             n++;
         }

@@ -165,14 +165,18 @@ struct Softmax {
     float m = -INFINITY, l = 0.0f;
     // sc: raw products (already times scale * log2 e); key of (kk, i) = key0 + 32 kk + 8 (i / 4) + 4 g + i % 4; keys past
     // `last` are not seen; returns the factor of what was accumulated so far
+    // MASKED: some key of the tile lies past `last`
+    template <bool MASKED>
     IT_DEV float step(v16f (&sc)[2], int key0, int g, int last, float pos, float slope2, h8 (&ph)[4], h8 (&pl)[4]) {
+        const float at = -slope2 * (pos - (float)(key0 + 4 * g));   // the bias of the lane's first key; the others are whole steps on
         float mt = -INFINITY;
 #pragma unroll
         for (int kk = 0; kk < 2; kk++)
 #pragma unroll
             for (int i = 0; i < 16; i++) {
-                const int key = key0 + 32 * kk + 8 * (i >> 2) + 4 * g + (i & 3);
-                const float v = key <= last ? fmaf(-slope2, pos - (float)key, sc[kk][i]) : -INFINITY;
+                const int off = 32 * kk + 8 * (i >> 2) + (i & 3);
+                float v = sc[kk][i] + fmaf(slope2, (float)off, at);
+                if (MASKED) v = key0 + 4 * g + off <= last ? v : -INFINITY;
                 sc[kk][i] = v;
                 mt = fmaxf(mt, v);
             }
@@ -270,7 +274,8 @@ __global__ __launch_bounds__(256) void attend_bias_split_k(BiasAttnP a, int n_sp
                 sc[kk] = __builtin_amdgcn_mfma_f32_32x32x16_f16(*(const h8*)(Ks + (32 * kk + c) * KS + 16 * s + 8 * g), qf, sc[kk], 0, 0, 0);
         }
         h8 ph[4], pl[4];
-        const float alpha = sm.step(sc, key0, g, k1 - 1, (float)pos, slope2, ph, pl);
+        const float alpha = key0 + KT <= k1 ? sm.step<false>(sc, key0, g, k1 - 1, (float)pos, slope2, ph, pl)
+                                            : sm.step<true>(sc, key0, g, k1 - 1, (float)pos, slope2, ph, pl);
         if (kt > 0) {
 #pragma unroll
             for (int dw = 0; dw < NDW; dw++)
@@ -369,7 +374,7 @@ __global__ __launch_bounds__(256) void attend_bias_batch_k(BiasAttnP a, int chun
     const int token = qt * QT + rt;
     const bool valid = rt < QT && token < a.n_q && rh < nh;
     const int head = kvh * G + first + (rh < nh ? rh : 0);
-    const int pos = valid ? base_pos + token : base_pos;   // (a row without a query sees the first tile's keys and is not stored)
+    const int pos = valid ? base_pos + token : base_pos;   // (a row without a query is not stored; it sees a key at least)
     const float slope2 = a.slopes ? a.slopes[head] * LOG2E : 0.0f;
     // the block's query rows, scaled, to LDS
     for (int i = tid; i < 128 * (HD / 4); i += 256) {
@@ -396,7 +401,6 @@ __global__ __launch_bounds__(256) void attend_bias_batch_k(BiasAttnP a, int chun
 #pragma unroll
         for (int i = 0; i < 16; i++) o[dt][i] = 0.0f;
     Softmax sm;
-    (void)first_pos;
     tile.fetch_k(0, a.n_pos);
     tile.fetch_v(0, a.n_pos);
     for (int kt = 0; kt < n_kt; kt++) {
@@ -421,7 +425,8 @@ __global__ __launch_bounds__(256) void attend_bias_batch_k(BiasAttnP a, int chun
             if ((s & 3) == 3) __builtin_amdgcn_sched_barrier(0);   // a few fragments in flight: registers are short
         }
         h8 ph[4], pl[4];
-        const float alpha = sm.step(sc, kt * KT, g, pos, (float)pos, slope2, ph, pl);
+        const float alpha = kt * KT + KT - 1 <= first_pos ? sm.step<false>(sc, kt * KT, g, pos, (float)pos, slope2, ph, pl)
+                                                          : sm.step<true>(sc, kt * KT, g, pos, (float)pos, slope2, ph, pl);
         if (__any(alpha != 1.0f)) {
 #pragma unroll
             for (int dt = 0; dt < ND; dt++)

@@ -21,16 +21,22 @@ template <> struct Raw8<W_F32> { uint4 a, b; };
 template <int FMT> IT_DEV const uint8_t* row_at(const uint8_t* w, int64_t row, int n_in) {
     return w + row * n_in * (FMT == W_F32 ? 4 : 2);
 }
+// a weight is read once a token: it need not stay in the caches
+typedef uint32_t u4 __attribute__((ext_vector_type(4)));
+IT_DEV uint4 stream16(const void* p) {
+    const u4 v = __builtin_nontemporal_load((const u4*)p);
+    return make_uint4(v.x, v.y, v.z, v.w);
+}
 // eight elements of a row from k on; AL: the row length is a multiple of 8 and the rows are 16-byte aligned
 template <int FMT, bool AL> IT_DEV Raw8<FMT> load8(const uint8_t* row, int k, int n_in) {
     Raw8<FMT> r{};
     if (AL) {
         if (k < n_in) {
             if constexpr (FMT == W_F32) {
-                r.a = *(const uint4*)((const float*)row + k);
-                r.b = *(const uint4*)((const float*)row + k + 4);
+                r.a = stream16((const float*)row + k);
+                r.b = stream16((const float*)row + k + 4);
             } else {
-                r.a = *(const uint4*)((const uint16_t*)row + k);
+                r.a = stream16((const uint16_t*)row + k);
             }
         }
     } else {
@@ -123,13 +129,21 @@ __global__ __launch_bounds__(256) void group_gemv_k(GroupP p, Groups gs) {
     // the input while the first rows are on their way
     {
         float ss = 0.0f;
-        for (int i = tid; i < n_ch * CH; i += 256) {
-            const float v = i < p.n_in ? p.x[i] : 0.0f;
-            ss = fmaf(v, v, ss);
-            xs[i] = v;
+        if (p.n_in % 4 == 0) {   // (device buffers are 16-byte aligned)
+            for (int i = tid * 4; i < n_ch * CH; i += 1024) {
+                const float4 v = i < p.n_in ? *(const float4*)(p.x + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+                ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+                *(float4*)(xs + i) = v;
+            }
+        } else {
+            for (int i = tid; i < n_ch * CH; i += 256) {
+                const float v = i < p.n_in ? p.x[i] : 0.0f;
+                ss = fmaf(v, v, ss);
+                xs[i] = v;
+            }
         }
         if (p.norm_w) {
-            ss = block_sum(ss, red);
+            ss = block_sum(ss, red);   // (its barriers also publish xs)
             const float rinv = 1.0f / sqrtf(ss / (float)p.n_in + p.eps);
             for (int i = tid; i < p.n_in; i += 256) xs[i] = xs[i] * rinv * p.norm_w[i];
         }
@@ -174,82 +188,121 @@ __global__ __launch_bounds__(256) void group_gemv_k(GroupP p, Groups gs) {
 }
 
 // ---------------------------------------------------------------- one token: sum of products into the residual
-template <int FMT, bool AL, int R>
-__global__ __launch_bounds__(256) void res_gemv_k(ResP p) {
-    extern __shared__ __align__(16) float xs[];   // the terms' inputs one behind the other, each padded to whole pieces
+// Eight waves a block, S of them on a group of R rows: the pieces of the terms' rows, one term behind the other, are dealt to
+// them in turn, and so sit in LDS: piece q of the inputs at q * CH.
+template <int FMT, bool AL, int R, int S>
+__global__ __launch_bounds__(512) void res_gemv_k(ResP p) {
+    constexpr int W = 8, UR = 8 / R;
+    extern __shared__ __align__(16) float xs[];
+    __shared__ float red[W], part_sum[W][R][RES_MAX];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int j0 = (blockIdx.x * 4 + wave) * R;
-    Raw8<FMT> w[R][U];
-    auto load = [&](const ResTerm& t, int c0) __attribute__((always_inline)) {
+    const int j0 = (blockIdx.x * (W / S) + wave / S) * R, s = wave % S;
+    const int n0 = (p.t[0].n_in + CH - 1) / CH, n1 = p.n_terms > 1 ? (p.t[1].n_in + CH - 1) / CH : 0, nq = n0 + n1;
+    const uint8_t* rp[RES_MAX][R];
 #pragma unroll
-        for (int u = 0; u < U; u++)
-#pragma unroll
-            for (int r = 0; r < R; r++) w[r][u] = load8<FMT, AL>(row_at<FMT>(t.w, min(j0 + r, p.n_out - 1), t.n_in), (c0 + u) * CH + lane * 8, t.n_in);
-    };
-    load(p.t[0], 0);
-    {
-        float* at = xs;
-        for (int k = 0; k < p.n_terms; k++) {
-            const int len = (p.t[k].n_in + CH - 1) / CH * CH;
-            for (int i = tid; i < len; i += 256) at[i] = i < p.t[k].n_in ? p.t[k].in[i] : 0.0f;
-            at += len;
-        }
-        __syncthreads();
-        at = xs;
-        for (int k = 0; k < p.n_terms; k++) {
-            const ResTerm& t = p.t[k];
-            if (t.norm_w) {
-                const int part = t.n_in / t.norm_groups;
-                for (int gi = wave; gi < t.norm_groups; gi += 4) {
-                    float ss = 0.0f;
-                    for (int i = lane; i < part; i += 64) ss = fmaf(at[gi * part + i], at[gi * part + i], ss);
-                    ss = group_sum<64>(ss);
-                    const float rinv = 1.0f / sqrtf(ss / (float)part + t.eps);
-                    for (int i = lane; i < part; i += 64) at[gi * part + i] = at[gi * part + i] * rinv * t.norm_w[gi * part + i];
-                }
-            }
-            at += (t.n_in + CH - 1) / CH * CH;
-        }
-        __syncthreads();
+    for (int r = 0; r < R; r++) {
+        const int j = min(j0 + r, p.n_out - 1);
+        rp[0][r] = row_at<FMT>(p.t[0].w, j, p.t[0].n_in);
+        rp[1][r] = n1 ? row_at<FMT>(p.t[1].w, j, p.t[1].n_in) : rp[0][r];
     }
-    if (j0 >= p.n_out) return;
-    float total[R];
+    Raw8<FMT> w[R][UR];
+    auto load = [&](int q0) __attribute__((always_inline)) {
 #pragma unroll
-    for (int r = 0; r < R; r++) total[r] = 0.0f;
-    const float* at = xs;
+        for (int u = 0; u < UR; u++) {
+            const int q = q0 + s + S * u;
+#pragma unroll
+            for (int r = 0; r < R; r++) {
+                if (q < n0) w[r][u] = load8<FMT, AL>(rp[0][r], q * CH + lane * 8, p.t[0].n_in);
+                else if (q < nq) w[r][u] = load8<FMT, AL>(rp[1][r], (q - n0) * CH + lane * 8, p.t[1].n_in);
+            }
+        }
+    };
+    load(0);
+    float* at = xs;
+    for (int k = 0; k < p.n_terms; k++) {
+        const int n = p.t[k].n_in, len = (n + CH - 1) / CH * CH;
+        const float* in = p.t[k].in;
+        if (n % 4 == 0) {   // (device buffers are 16-byte aligned)
+            for (int i = tid * 4; i < len; i += 2048) *(float4*)(at + i) = i < n ? *(const float4*)(in + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+        } else {
+            for (int i = tid; i < len; i += 512) at[i] = i < n ? in[i] : 0.0f;
+        }
+        at += len;
+    }
+    at = xs;
     for (int k = 0; k < p.n_terms; k++) {
         const ResTerm& t = p.t[k];
-        const int n_ch = (t.n_in + CH - 1) / CH;
-        float acc[R];
-#pragma unroll
-        for (int r = 0; r < R; r++) acc[r] = 0.0f;
-        for (int c0 = 0; c0 < n_ch; c0 += U) {
-            if (k > 0 || c0 > 0) load(t, c0);
-#pragma unroll
-            for (int u = 0; u < U; u++) {
-                if (c0 + u < n_ch) {
-                    const float4 x0 = *(const float4*)(at + (c0 + u) * CH + lane * 8), x1 = *(const float4*)(at + (c0 + u) * CH + lane * 8 + 4);
-                    const float x[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
-#pragma unroll
-                    for (int r = 0; r < R; r++) {
-                        float f[8];
-                        widen8<FMT>(w[r][u], f);
-#pragma unroll
-                        for (int e = 0; e < 8; e++) acc[r] = fmaf(f[e], x[e], acc[r]);
-                    }
+        if (t.norm_w) {   // a part of the row to one, two, four or all eight waves
+            const int part = t.n_in / t.norm_groups, wpg = t.norm_groups > 4 ? 1 : t.norm_groups > 2 ? 2 : t.norm_groups > 1 ? 4 : 8;
+            __syncthreads();
+            for (int g0 = 0; g0 < t.norm_groups; g0 += W / wpg) {
+                const int gi = g0 + wave / wpg, sub = wave % wpg;
+                float* a = at + gi * part;
+                float ss = 0.0f;
+                if (gi < t.norm_groups)
+                    for (int i = sub * 64 + lane; i < part; i += 64 * wpg) ss = fmaf(a[i], a[i], ss);
+                ss = group_sum<64>(ss);
+                if (wpg > 1) {
+                    if (lane == 0) red[wave] = ss;
+                    __syncthreads();
+                    ss = 0.0f;
+                    for (int i = 0; i < wpg; i++) ss += red[wave - sub + i];
                 }
+                const float rinv = 1.0f / sqrtf(ss / (float)part + t.eps);
+                if (gi < t.norm_groups)
+                    for (int i = sub * 64 + lane; i < part; i += 64 * wpg) a[i] = a[i] * rinv * t.norm_w[gi * part + i];
             }
         }
-        at += n_ch * CH;
+        at += (t.n_in + CH - 1) / CH * CH;
+    }
+    __syncthreads();
+    float acc[RES_MAX][R];
 #pragma unroll
-        for (int r = 0; r < R; r++) {
-            acc[r] = group_sum<64>(acc[r]);
-            total[r] += t.scale ? acc[r] * t.scale[min(j0 + r, p.n_out - 1)] : acc[r];
+    for (int k = 0; k < RES_MAX; k++)
+#pragma unroll
+        for (int r = 0; r < R; r++) acc[k][r] = 0.0f;
+    for (int q0 = 0; q0 < nq; q0 += S * UR) {
+        if (q0) load(q0);
+#pragma unroll
+        for (int u = 0; u < UR; u++) {
+            const int q = q0 + s + S * u;
+            if (q >= nq) continue;
+            const float4 x0 = *(const float4*)(xs + q * CH + lane * 8), x1 = *(const float4*)(xs + q * CH + lane * 8 + 4);
+            const float x[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
+#pragma unroll
+            for (int r = 0; r < R; r++) {
+                float f[8], v = q < n0 ? acc[0][r] : acc[1][r];
+                widen8<FMT>(w[r][u], f);
+#pragma unroll
+                for (int e = 0; e < 8; e++) v = fmaf(f[e], x[e], v);
+                if (q < n0) acc[0][r] = v;
+                else acc[1][r] = v;
+            }
         }
     }
 #pragma unroll
-    for (int r = 0; r < R; r++)
-        if (lane == r && j0 + r < p.n_out) p.x[j0 + r] += total[r];
+    for (int k = 0; k < RES_MAX; k++)
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            acc[k][r] = group_sum<64>(acc[k][r]);
+            if (S > 1 && lane == 0) part_sum[wave][r][k] = acc[k][r];
+        }
+    if (S > 1) __syncthreads();
+    if (s) return;
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        if (lane != r || j0 + r >= p.n_out) continue;
+        float total = 0.0f;
+        for (int k = 0; k < p.n_terms; k++) {
+            float v = k ? acc[1][r] : acc[0][r];
+            if (S > 1) {
+                v = 0.0f;
+                for (int i = 0; i < S; i++) v += part_sum[wave + i][r][k];
+            }
+            total += p.t[k].scale ? v * p.t[k].scale[j0 + r] : v;
+        }
+        p.x[j0 + r] += total;
+    }
 }
 
 // ---------------------------------------------------------------- a few tokens
@@ -334,14 +387,16 @@ __global__ __launch_bounds__(256) void norm_rows_k(const float* __restrict__ x, 
     if (out16 && g == groups - 1 && tid < pad8(nd) - nd) out16[row * pad8(nd) + nd + tid] = 0;
 }
 
-// rows of whole float4s and one part: a thread keeps its pieces between the two passes (up to 8,192 elements)
+// parts of whole float4s, rows of whole 16-byte bf16 pieces: a thread keeps its pieces between the two passes (up to 8,192
+// elements a part)
 template <int V>
-__global__ __launch_bounds__(256) void norm_rows4_k(const float* __restrict__ x, const float* __restrict__ w, float eps, int nd,
+__global__ __launch_bounds__(256) void norm_rows4_k(const float* __restrict__ x, const float* __restrict__ w, float eps, int part,
                                                     float* __restrict__ out32, uint16_t* __restrict__ out16) {
     __shared__ float red[4];
-    const int tid = threadIdx.x, n4 = nd >> 2;
-    const int64_t row = blockIdx.x;
-    const float4* xr = (const float4*)(x + row * nd);
+    const int tid = threadIdx.x, n4 = part >> 2;
+    const int64_t at0 = ((int64_t)blockIdx.x * gridDim.y + blockIdx.y) * part;   // rows are `gridDim.y` parts
+    const float4* xr = (const float4*)(x + at0);
+    w += blockIdx.y * part;
     float4 v[V];
     float ss = 0.0f;
 #pragma unroll
@@ -351,16 +406,16 @@ __global__ __launch_bounds__(256) void norm_rows4_k(const float* __restrict__ x,
         ss = fmaf(v[i].x, v[i].x, fmaf(v[i].y, v[i].y, fmaf(v[i].z, v[i].z, fmaf(v[i].w, v[i].w, ss))));
     }
     ss = block_sum(ss, red);
-    const float rinv = 1.0f / sqrtf(ss / (float)nd + eps);
+    const float rinv = 1.0f / sqrtf(ss / (float)part + eps);
 #pragma unroll
     for (int i = 0; i < V; i++) {
         const int at = tid + i * 256;
         if (at >= n4) continue;
         const float4 ww = ((const float4*)w)[at];
         const float4 r = make_float4(v[i].x * rinv * ww.x, v[i].y * rinv * ww.y, v[i].z * rinv * ww.z, v[i].w * rinv * ww.w);
-        if (out32) ((float4*)(out32 + row * nd))[at] = r;
+        if (out32) ((float4*)(out32 + at0))[at] = r;
         if (out16)
-            ((uint2*)(out16 + row * nd))[at] = make_uint2(to_bf16(r.x) | ((uint32_t)to_bf16(r.y) << 16), to_bf16(r.z) | ((uint32_t)to_bf16(r.w) << 16));
+            ((uint2*)(out16 + at0))[at] = make_uint2(to_bf16(r.x) | ((uint32_t)to_bf16(r.y) << 16), to_bf16(r.z) | ((uint32_t)to_bf16(r.w) << 16));
     }
 }
 
@@ -444,17 +499,23 @@ template <int FMT, bool AL> bool launch_group(const GroupP& p, hipStream_t s) {
     }
     return true;
 }
+// about one block a CU and eight rows in the making in it: rows shared by several waves where there are few, several rows a
+// wave where there are many
 template <int FMT, bool AL> bool launch_res(const ResP& p, hipStream_t s) {
     size_t lds = 0;
     for (int i = 0; i < p.n_terms; i++) lds += padded(p.t[i].n_in) * sizeof(float);
-    if (p.n_out >= 8192) {
-        if (!allow_lds(res_gemv_k<FMT, AL, 2>, lds)) return false;
-        hipLaunchKernelGGL((res_gemv_k<FMT, AL, 2>), dim3((p.n_out + 7) / 8), dim3(256), lds, s, p);
-    } else {
-        if (!allow_lds(res_gemv_k<FMT, AL, 1>, lds)) return false;
-        hipLaunchKernelGGL((res_gemv_k<FMT, AL, 1>), dim3((p.n_out + 3) / 4), dim3(256), lds, s, p);
-    }
-    return true;
+#define IT_RES(R, S)                                                                                        \
+    do {                                                                                                    \
+        if (!allow_lds(res_gemv_k<FMT, AL, R, S>, lds)) return false;                                       \
+        const int per = 8 / S * R;                                                                          \
+        hipLaunchKernelGGL((res_gemv_k<FMT, AL, R, S>), dim3((p.n_out + per - 1) / per), dim3(512), lds, s, p); \
+        return true;                                                                                        \
+    } while (0)
+    if (p.n_out <= 512) IT_RES(1, 4);
+    if (p.n_out <= 1024) IT_RES(1, 2);
+    if (p.n_out <= 2048) IT_RES(1, 1);
+    IT_RES(2, 1);
+#undef IT_RES
 }
 
 // one call per (format, alignment)
@@ -511,11 +572,13 @@ void res_rows(const ResP& p, hipStream_t s) {
 
 void norm_rows(const float* x, const float* w, int groups, float eps, int64_t n_rows, int nd, float* out32, uint16_t* out16, hipStream_t s) {
     if (n_rows <= 0) return;
-    if (w && groups == 1 && nd % 8 == 0 && nd <= 8192 && aligned16(x) && aligned16(w) && aligned16(out32) && aligned16(out16)) {
-        if (nd <= 1024) hipLaunchKernelGGL(norm_rows4_k<1>, dim3((unsigned)n_rows), dim3(256), 0, s, x, w, eps, nd, out32, out16);
-        else if (nd <= 2048) hipLaunchKernelGGL(norm_rows4_k<2>, dim3((unsigned)n_rows), dim3(256), 0, s, x, w, eps, nd, out32, out16);
-        else if (nd <= 4096) hipLaunchKernelGGL(norm_rows4_k<4>, dim3((unsigned)n_rows), dim3(256), 0, s, x, w, eps, nd, out32, out16);
-        else hipLaunchKernelGGL(norm_rows4_k<8>, dim3((unsigned)n_rows), dim3(256), 0, s, x, w, eps, nd, out32, out16);
+    const int part = nd / groups;
+    if (w && nd % 8 == 0 && part % 4 == 0 && part <= 8192 && aligned16(x) && aligned16(w) && aligned16(out32) && aligned16(out16)) {
+        const dim3 grid((unsigned)n_rows, groups);
+        if (part <= 1024) hipLaunchKernelGGL(norm_rows4_k<1>, grid, dim3(256), 0, s, x, w, eps, part, out32, out16);
+        else if (part <= 2048) hipLaunchKernelGGL(norm_rows4_k<2>, grid, dim3(256), 0, s, x, w, eps, part, out32, out16);
+        else if (part <= 4096) hipLaunchKernelGGL(norm_rows4_k<4>, grid, dim3(256), 0, s, x, w, eps, part, out32, out16);
+        else hipLaunchKernelGGL(norm_rows4_k<8>, grid, dim3(256), 0, s, x, w, eps, part, out32, out16);
         return;
     }
     hipLaunchKernelGGL(norm_rows_k, dim3((unsigned)n_rows, groups), dim3(256), 0, s, x, w, groups, eps, nd, out32, out16);

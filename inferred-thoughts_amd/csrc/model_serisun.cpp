@@ -69,7 +69,7 @@ struct Run {
 
 struct Serisun : it_model {
     its::File file;
-    uint64_t n_vocab = 0, nd = 0;
+    uint64_t n_vocab = 0, nd = 0, passes = 1;   // passes: through the looped layers
     float eps = 0, logit_scale = 1;
     std::vector<Layer> layers;
     std::vector<Run> runs;
@@ -139,6 +139,7 @@ struct Serisun : it_model {
             if (!size(loop, "loop", "start", &a, 0) || !size(loop, "loop", "stop", &b) || !size(loop, "loop", "times", &times)) return false;
             if (a >= b || b > layers.size() || times > 4096) return fail("config.json: loop does not name a stretch of the layers");
         }
+        passes = times;
         auto add = [&](uint64_t i, int64_t opens) { runs.push_back(Run{i, opens, layers[i].attention ? kv++ : st++}); };
         for (uint64_t i = 0; i < a; i++) add(i, -1);
         for (uint64_t t = 0; looped && t < times; t++)
@@ -241,7 +242,7 @@ struct SerisunEngine : it_engine {
     std::vector<HostBuf*> buffers() override { return {&emb, &x, &q, &attn, &u, &y, &ff, &last, &picked}; }
 
     void fit(uint64_t n) {
-        emb.fit(n * m->nd, be);
+        if (m->passes > 1) emb.fit(n * m->nd, be);
         x.fit(n * m->nd, be);
         for (const Layer& l : m->layers) {
             if (l.attention) {
@@ -329,8 +330,9 @@ struct SerisunEngine : it_engine {
         const uint64_t nd = m->nd;
         it_hip_begin_pass(be, n);
         fit(n);
-        if (int rc = embed(tokens, n, emb.p(), ring_index)) return rc;
-        it_hip_gather_chunks(be, emb.p(), n * nd, n * nd, n * nd, 0, x.p(), n * nd);
+        // the embedding is kept beside the residual where a later pass of the loop adds it again
+        if (int rc = embed(tokens, n, m->passes > 1 ? emb.p() : x.p(), ring_index)) return rc;
+        if (m->passes > 1) it_hip_gather_chunks(be, emb.p(), n * nd, n * nd, n * nd, 0, x.p(), n * nd);
         tr("inp_embd", 0, x, n * nd);
         for (uint64_t i = 0; i < m->runs.size(); i++) {
             const Run& r = m->runs[i];

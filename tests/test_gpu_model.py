@@ -275,3 +275,45 @@ def test_checkpoint_restore_continues_identically(tiny_gguf, exact):
         oe.close(); om.close()
     assert be.take_error() is None
     e.close(); m.close(); be.close()
+
+
+def test_logits_of_chosen_rows(hip, tiny_gguf):
+    """forward_rows: the rows' logits are those of passes that end there, whatever else is asked for and however the engine's
+    batch cuts the tokens."""
+    import inferred_hip as ih
+    hip.drop_mirrors()
+    t = prompt_ids(40, seed=4)
+    m = ih.Model(tiny_gguf)
+    e = ih.Engine(m, hip, 64, 16)
+    want = {}
+    for n in (1, 4, 16, 17, 40):
+        e.reset()
+        want[n - 1] = e.prefill(t[:n])
+    for rows in ([0, 3, 15, 16, 39], [39], []):
+        e.reset()
+        got = e.forward_rows(t, rows)
+        assert e.pos == 40 and got.shape == (len(rows), m.n_vocab)
+        for r, g in zip(rows, got):
+            assert_bits_equal(g, want[r])
+    e.close(); m.close()
+
+
+def test_the_trace_runner_on_a_gguf_file(tiny_gguf, tmp_path):
+    import json
+    import subprocess
+    from pathlib import Path
+    import inferred_hip as ih
+    run = str(Path(__file__).resolve().parent.parent / "bin" / "trace_run")
+    t = prompt_ids(20, seed=6)
+    steps = [{"step": 0, "entries": [{"id": "x", "tokens": [int(i) for i in t[:19]], "want": [18]}]},
+             {"step": 1, "entries": [{"id": "x", "tokens": [int(t[19])], "want": [0]}], "end": ["x"]}]
+    p = subprocess.run([run, "--model", str(tiny_gguf), "--dtype", "bfloat16", "--out", str(tmp_path), "--max-tokens", "20"],
+                       input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True, text=True, timeout=90)
+    assert p.returncode == 0, p.stderr[-2000:]
+    be = ih.Hip(); m = ih.Model(tiny_gguf); e = ih.Engine(m, be, 20, 2048)
+    for k, part in enumerate((t[:19], t[19:])):
+        assert _rel(np.fromfile(tmp_path / f"{k}.f32", "<f4"), e.forward(part)) < 1e-5
+    e.close(); m.close(); be.close()
+    p = subprocess.run([run, "--model", str(tiny_gguf), "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", "20"],
+                       input="", capture_output=True, text=True, timeout=90)
+    assert p.returncode == 3 and "no 32-bit form" in p.stderr
