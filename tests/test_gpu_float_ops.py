@@ -358,6 +358,24 @@ def test_mamba2_where_tokens_forget_almost_everything(be, n):
     assert rel(m.run(be, u, 0), want) < 1e-4 and rel(m.read_state(be), S) < 1e-4
 
 
+def test_mamba2_over_more_chunks_than_are_taken_at_once(be):
+    """A state so large that the chunked form takes eight chunks at a time: one call of ten against two calls of fewer."""
+    r = rng(2)
+    m = Mixer(r, 128, 64, 512, 1, 2)
+    u = 0.5 * r.standard_normal((600, m.ud)).astype(np.float32)
+    runs = []
+    for pieces in ((600,), (300, 300)):
+        at, out = 0, []
+        for c in pieces:
+            out.append(m.run(be, u[at:at + c], at))
+            at += c
+        runs.append((np.concatenate(out), m.read_state(be)))
+        for b in (m.ring, m.state):
+            b[:] = 0
+            be.L.it_hip_zero_slab(be.h, b.ctypes.data)
+    assert rel(runs[0][0], runs[1][0]) < 1e-4 and rel(runs[0][1], runs[1][1]) < 1e-4 and np.abs(runs[0][1]).max() > 0.1
+
+
 # ---------------------------------------------------------------- the small ones
 @pytest.mark.parametrize("ff", [24, 21])
 def test_rows_left_in_bf16_are_read_as_f32_where_an_op_needs_them(be, ff):
