@@ -321,7 +321,9 @@ int it_hip_mfma_ceiling(it_hip*, int kind, int iters, double* ops_per_s);
  * batch size from the buffer lengths; first error kept.  Each op is one sublayer step and picks its form by the batch: one
  * token a fused launch, up to 16 tokens a few, more tokens the bf16 matrix cores (bf16 matrices, and not in 32-bit mode:
  * IT_HIP_F32 and IT_HIP_EXACT take 32-bit kernels throughout).  With IT_HIP_NO_FUSE every step of an op is a launch. */
-/* One matrix of a group that reads the same activations.  `up` (data non-NULL) makes it a gated pair: silu(w x) * (up x).
+#define IT_ACT_SILU 0u
+#define IT_ACT_RELU 1u
+/* One matrix of a group that reads the same activations.  `up` (data non-NULL) makes it a gated pair: act(w x) * (up x).
  * The rows go to `out` (times `scale`), or, with `slab` set, to rows slab_row .. of a cache slab whose elements are f16 (f32
  * in 32-bit mode): heads of head_dim elements, head_stride elements apart, n_out / head_dim of them a row. */
 typedef struct {
@@ -332,11 +334,23 @@ typedef struct {
     uint64_t slab_len; /* elements */
     uint64_t slab_row, head_dim, head_stride;
     float scale;
-    uint32_t _pad;
+    uint32_t act; /* of w where up is given: IT_ACT_* */
 } it_group_mat;
 /* out_m = scale_m * W_m h, h = RMS norm of x times norm_w (norm_w NULL: h = x); at most 6 matrices of n_in = row length */
 void it_hip_norm_matmuls(it_hip*, const float* x, uint64_t x_len, const float* norm_w, uint64_t n_in, float eps,
                          const it_group_mat* mats, uint64_t n_mats);
+/* What a sublayer whose output is normed adds to the residual: x_new = x + mult * (RMS norm of y times norm_w), rows as x;
+ * x_new is another buffer than x */
+typedef struct {
+    const float* y;
+    const float* norm_w;
+    float* x_new;
+    float eps, mult;
+} it_add_normed;
+void it_hip_add_normed(it_hip*, const float* x, uint64_t x_len, const it_add_normed* add, uint64_t n_in);
+/* it_hip_add_normed, then it_hip_norm_matmuls of x_new */
+void it_hip_add_norm_matmuls(it_hip*, const float* x, uint64_t x_len, const it_add_normed* add, const float* norm_w, uint64_t n_in, float eps,
+                             const it_group_mat* mats, uint64_t n_mats);
 /* One term of a residual sum: scale (elementwise, NULL: 1) times W applied to `in`, whose rows are first, when norm_w is
  * set, cut into norm_groups equal parts, each divided by its own root mean square, and multiplied by norm_w. */
 typedef struct {
@@ -347,14 +361,19 @@ typedef struct {
     const float* norm_w;
     uint64_t norm_groups;
     float eps;
-    uint32_t _pad;
+    uint32_t norm_shared; /* 1: norm_w has one part's elements, used for every part */
+    const float* gate;    /* rows as `in`, NULL: none; only with norm_w: the normed input times silu(gate) */
+    uint64_t gate_len;
 } it_res_term;
 /* x += sum of at most 2 terms; the terms are added up before x is */
 void it_hip_matmul_residual(it_hip*, float* x, uint64_t x_len, const it_res_term* terms, uint64_t n_terms);
+/* out = that sum */
+void it_hip_matmul_sum(it_hip*, float* out, uint64_t out_len, const it_res_term* terms, uint64_t n_terms);
 /* Causal attention of the last n_q of n_pos positions over slabs written by it_hip_norm_matmuls:
  *   score = (q . k) * scale * temp(position) - slopes[head] * (position - key), slopes NULL: no bias;
  *   temp(p) = 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1), temp_coef 0: none;
- *   weights = exp(score) / (sink + sum exp(score)), sink 0 or 1; query head h reads KV head h / (n_head / n_head_kv) */
+ *   weights = exp(score) / (sink * exp(sinks[head]) + sum exp(score)), sink 0 or 1, sinks NULL: all 0;
+ *   window w > 0: position i sees the keys i - w + 1 .. i; query head h reads KV head h / (n_head / n_head_kv) */
 typedef struct {
     const float* q;
     uint64_t q_len;
@@ -366,6 +385,8 @@ typedef struct {
     const float* slopes;
     float temp_coef;
     uint32_t temp_every;
+    const float* sinks;
+    uint64_t window;
 } it_attn_bias;
 void it_hip_attend_bias(it_hip*, const it_attn_bias* a, float* out, uint64_t out_len);
 /* The Mamba-2 mixer between its projections: u rows are [z | x | B | C | dt] (inner, inner, groups * n, groups * n, heads;
@@ -378,6 +399,50 @@ typedef struct {
 } it_mamba2;
 void it_hip_mamba2(it_hip*, const it_mamba2* m, const float* u, uint64_t u_len, float* conv_ring, uint64_t ring_len, float* state,
                    uint64_t state_len, float* out, uint64_t out_len);
+/* Gated linear attention between its projections, per head and token:
+ *   alpha = sigmoid(a2 low + a2_b)^(1 / tau), a factor per key channel;  S = diag(alpha) S + k v^T;  out = S^T q
+ * q, k rows of heads * dim, v and out rows of heads * vdim, low rows of a2.n_in; a2 [heads * dim][rank]; state [heads][vdim][dim] */
+typedef struct {
+    const float *q, *k, *v, *low;
+    uint64_t q_len, k_len, v_len, low_len;
+    it_weights a2;
+    const float* a2_b;
+    uint64_t heads, dim, vdim;
+    float tau;
+    uint32_t _pad;
+} it_gla;
+void it_hip_gla(it_hip*, const it_gla* g, float* state, uint64_t state_len, float* out, uint64_t out_len);
+/* Rotary positions on neighbouring dimensions (2i, 2i + 1), the first `dims`: angle p * f_i, f_i = base^(-2i / dims).  factor > 0:
+ * with ramp_i from 0 (as many turns over `original` positions as `fast`) to 1 (`slow`), f_i becomes f_i (1 - ramp_i + ramp_i / factor),
+ * and cos and sin are multiplied by 0.1 ln(factor) + 1. */
+typedef struct {
+    double base;
+    uint64_t dims;
+    double factor, original, fast, slow;
+} it_rope;
+/* Latent attention between its projections, over a cache slab of rows [latent (rank) | rotated key part (rot_dim)], padded to a
+ * multiple of 8 elements, one for all heads.
+ *   kv rows [latent | key part]: the latent's RMS norm times kv_norm and the rotated key part become the rows pos ..;
+ *     NULL: these rows are there already (another layer's)
+ *   q rows of heads * (dim + rot_dim), [unrotated | rotated] a head, not yet rotated (the call may leave them rotated)
+ *   score = (q_unrotated . uk_h c + q_rotated . k_rotated) * scale over the window (0: all positions up to the query's)
+ *   out_h = sigmoid(gate_h) * sum of weights * uv_h c, weights = exp(score) / (exp(sinks[h]) + sum exp(score))
+ * sinks NULL: no sink; gate NULL: no gate; uk [heads * dim][rank], uv [heads * vdim][rank]; `pos`: of the first token */
+typedef struct {
+    float* q;
+    const float* kv;
+    uint64_t q_len, kv_len;
+    const float* kv_norm;
+    void* slab;
+    uint64_t slab_len; /* elements */
+    it_weights uk, uv;
+    const float *sinks, *gate;
+    uint64_t gate_len;
+    uint64_t heads, dim, rot_dim, vdim, rank, pos, window;
+    float scale, eps;
+    it_rope rope;
+} it_attn_latent;
+void it_hip_attend_latent(it_hip*, const it_attn_latent* a, float* out, uint64_t out_len);
 /* x[t] += rows[t] (NULL: none), then + vec (NULL: none) */
 void it_hip_add_rows(it_hip*, float* x, uint64_t x_len, const float* rows, const float* vec, uint64_t vec_len);
 /* out = the rows `idx` of src (rows of `width` floats) */
@@ -416,7 +481,7 @@ typedef struct it_model it_model;
 typedef struct it_engine it_engine;
 typedef void (*it_trace_fn)(void* user, const char* name, uint32_t layer, const float* data, uint64_t n);
 
-/* `path`: a GGUF file (qwen35moe), or a folder with config.json and model.safetensors (Serisun); the design is chosen by the
+/* `path`: a GGUF file (qwen35moe), or a folder with config.json and model.safetensors (Serisun, Nubedra); the design is chosen by the
  * architecture name the file or the configuration gives */
 it_model* it_model_open(const char* path, char* err, size_t err_len);
 void it_model_close(it_model*);

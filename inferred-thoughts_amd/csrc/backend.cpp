@@ -919,20 +919,45 @@ bool it_hip::route_stage(const it_route* r, const int32_t** ids, const float** w
 const float2* it_hip::rope_table(float theta, uint64_t n_rot, uint64_t need_pos) {
     uint32_t tb;
     memcpy(&tb, &theta, 4);
-    uint64_t key = ((uint64_t)tb << 32) | n_rot;
+    return rope_table_of(((uint64_t)tb << 32) | n_rot, n_rot / 2, need_pos, [&](std::vector<double>& freq) {
+        for (size_t i = 0; i < freq.size(); i++) freq[i] = pow((double)theta, -2.0 * (double)i / (double)n_rot);
+        return 1.0;
+    });
+}
+const float2* it_hip::rope_table(const it_rope& r, uint64_t need_pos) {
+    uint64_t key = 0xcbf29ce484222325ull;   // (the top bit keeps it apart from the plain tables')
+    for (double v : {r.base, (double)r.dims, r.factor, r.original, r.fast, r.slow}) {
+        uint64_t u;
+        memcpy(&u, &v, 8);
+        for (int b = 0; b < 64; b += 8) key = (key ^ ((u >> b) & 0xff)) * 0x100000001b3ull;
+    }
+    return rope_table_of(key | (1ull << 63), r.dims / 2, need_pos, [&](std::vector<double>& freq) {
+        const double d = (double)r.dims;
+        for (size_t i = 0; i < freq.size(); i++) freq[i] = pow(r.base, -2.0 * (double)i / d);
+        if (!(r.factor > 0)) return 1.0;
+        auto dim_of = [&](double turns) { return d * log(r.original / (2.0 * M_PI * turns)) / (2.0 * log(r.base)); };
+        const double lo = std::max(floor(dim_of(r.fast)), 0.0), hi = std::min(ceil(dim_of(r.slow)), d - 1.0);
+        for (size_t i = 0; i < freq.size(); i++) {
+            const double ramp = std::min(std::max(((double)i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+            freq[i] = freq[i] / r.factor * ramp + freq[i] * (1.0 - ramp);
+        }
+        return 0.1 * log(r.factor) + 1.0;
+    });
+}
+// `fill` sets the frequencies and returns the factor of cos and sin
+const float2* it_hip::rope_table_of(uint64_t key, size_t half, uint64_t need_pos, const std::function<double(std::vector<double>&)>& fill) {
     Rope& r = ropes[key];
     if (r.cap_pos >= need_pos) return r.dev;
     need_eager("the rope table has to grow");
     size_t cap = r.cap_pos ? r.cap_pos : 8192;
     while (cap < need_pos) cap *= 2;
-    size_t half = n_rot / 2;
-    std::vector<float2> tab(cap * half);
     std::vector<double> freq(half);
-    for (size_t i = 0; i < half; i++) freq[i] = pow((double)theta, -2.0 * (double)i / (double)n_rot);
+    const double mult = fill(freq);
+    std::vector<float2> tab(cap * half);
     for (size_t p = 0; p < cap; p++)
         for (size_t i = 0; i < half; i++) {
             double th = (double)p * freq[i];
-            tab[p * half + i] = make_float2((float)cos(th), (float)sin(th));
+            tab[p * half + i] = make_float2((float)(mult * cos(th)), (float)(mult * sin(th)));
         }
     float2* dev = nullptr;
     if (!check(hipMalloc((void**)&dev, tab.size() * sizeof(float2)), "hipMalloc(rope table)")) return nullptr;
@@ -2488,7 +2513,7 @@ int it_hip_profile_end(it_hip* be, it_profile_row* rows, int max_rows) {
                                                    "gdn_rows (l2 norm + delta rule)", "attn_prep (norm + rope + kv write)",
                                                    "layer_chain (a run of layers, persistent)",
                                                    "group (norm + unquantized matrices)",
-                                                   "residual (matrices + residual sum)", "mamba2 (conv + state space)"};
+                                                   "residual (matrices + residual sum)", "mamba2 (conv + state space)", "gla (gated linear attention)"};
     be->prof_on = false;
     be->check(hipStreamSynchronize(be->stream), "sync");
     it_profile_row acc[it_hip::FAM_COUNT];

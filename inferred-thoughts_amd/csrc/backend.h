@@ -44,7 +44,8 @@
 enum OpId : int {
     OP_RMS = 1, OP_RMS_HEADS, OP_L2, OP_MATMUL, OP_ROPE, OP_SOFTMAX, OP_ATTEND, OP_EW, OP_SCALE, OP_CONV, OP_GATHER,
     OP_SCATTER, OP_DELTA, OP_ROUTE, OP_EXPERTS, OP_GLU, OP_FINISH, OP_ROWS, OP_SIGADD, OP_KVWRITE, OP_EMBED,
-    OP_GROUP, OP_RESIDUAL, OP_ATTEND_BIAS, OP_MAMBA2, OP_ADD_ROWS, OP_GATHER_ROWS,   // unquantized models: issued as they are
+    OP_GROUP, OP_RESIDUAL, OP_ATTEND_BIAS, OP_MAMBA2, OP_ADD_ROWS, OP_GATHER_ROWS,
+    OP_ADD_NORMED, OP_GLA, OP_ATTEND_LATENT,   // unquantized models: issued as they are
     OP_QUANT = 101
 };
 
@@ -94,9 +95,10 @@ struct it_hip {
     uint16_t* act_half_reserve(Act& a, size_t rows, size_t row);
     const uint16_t* act_half_if_valid(const float* host, size_t rows, size_t row);
     void act_widen(Act& a);                  // the f32 mirror of rows that exist in bf16 only
+    bool add_in(const float* x, uint64_t x_len, const it_add_normed& a, uint64_t n_in, itk::AddNormed* out);
     // scratch of the unquantized ops, by use: f32 rows, bf16 rows
     struct Tmp { void* p = nullptr; size_t bytes = 0; };
-    Tmp tmps[6];
+    Tmp tmps[11];
     void* tmp_for(int which, size_t bytes);
     Act* act_by_dev(const void* dev);        // the mirror whose device buffer holds `dev`, or null
     bool held_touches(const void* dev, size_t bytes) const;   // an op held back reads or writes inside [dev, dev + bytes)
@@ -208,6 +210,8 @@ struct it_hip {
     };
     std::unordered_map<uint64_t, Rope> ropes;
     const float2* rope_table(float theta, uint64_t n_rot, uint64_t need_pos);
+    const float2* rope_table(const it_rope& r, uint64_t need_pos);   // scaled frequencies, cos and sin times their factor
+    const float2* rope_table_of(uint64_t key, size_t half, uint64_t need_pos, const std::function<double(std::vector<double>&)>& fill);
 
     // ---- scratch
     float* attn_scratch = nullptr;
@@ -368,7 +372,7 @@ struct it_hip {
 
     // ---- per-kernel-family timing with HIP events on the launch stream
     enum Family { FAM_MATMUL = 0, FAM_MOE_GLU, FAM_MOE_DOWN, FAM_DELTA, FAM_ATTEND, FAM_NORM, FAM_ROUTER, FAM_OTHER,
-                  FAM_FUSED_GEMV, FAM_LM_HEAD, FAM_GDN_ROWS, FAM_ATTN_PREP, FAM_CHAIN, FAM_GROUP, FAM_RESIDUAL, FAM_SSD, FAM_COUNT };
+                  FAM_FUSED_GEMV, FAM_LM_HEAD, FAM_GDN_ROWS, FAM_ATTN_PREP, FAM_CHAIN, FAM_GROUP, FAM_RESIDUAL, FAM_SSD, FAM_GLA, FAM_COUNT };
     struct ProfSpan {
         hipEvent_t a, b;
         int fam;

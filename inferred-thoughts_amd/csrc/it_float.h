@@ -11,6 +11,9 @@ IT_DEV uint16_t to_bf16(float f) { return __builtin_bit_cast(uint16_t, (__bf16)f
 IT_DEV float silu_exact(float z) { return z / (1.0f + expf(-z)); }
 IT_DEV float softplus_exact(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
 
+IT_DEV float sigmoid_exact(float z) { return 1.0f / (1.0f + expf(-z)); }
+IT_DEV float act_of(int act, float z) { return act == ACT_RELU ? fmaxf(z, 0.0f) : silu_exact(z); }
+
 IT_DEV void group_store(const GroupMat& m, int t, int j, float v) {
     v *= m.scale;
     const GroupOut& o = m.o;

@@ -1,8 +1,9 @@
 // Attention with what the kernels of k_attn.hip and k_attn_prefill.hip do not have: a distance bias per head
-// (score -= slope * (i - j)), a sink in the softmax's denominator (1 + sum exp(score)), a query temperature that grows
-// with the position, and keys and values of different, arbitrary sizes.
+// (score -= slope * (i - j)), a sink in the softmax's denominator (e^sink_h + sum exp(score)), a query temperature that grows
+// with the position, a sliding window, and keys and values of different, arbitrary sizes.
 //
-//     score_ij = (temp(i) q_i . k_j) * scale - slope * (i - j),  j <= i;   out_i = sum_j exp(score_ij) v_j / (sink + sum_j exp(score_ij))
+//     score_ij = (temp(i) q_i . k_j) * scale - slope * (i - j),  i - window < j <= i
+//     out_i = sum_j exp(score_ij) v_j / (e^sink_h + sum_j exp(score_ij))
 //
 // The heads of a cache row are k_stride (v_stride) elements apart, a multiple of eight with zeros behind the head's own
 // elements, so that every 16-byte piece of a row is aligned whatever the head size.
@@ -38,6 +39,12 @@ IT_DEV float temperature(const BiasAttnP& a, int pos) {
     return 1.0f + a.temp_coef * logf((float)((pos + 1) / a.temp_every + 1));
 }
 
+IT_DEV int first_seen(const BiasAttnP& a, int pos) { return a.window ? max(0, pos - a.window + 1) : 0; }
+// the sink in the log2 domain, ahead of a maximum
+IT_DEV float sink_share(const BiasAttnP& a, int head, float m) {
+    return a.sink ? __builtin_amdgcn_exp2f((a.sinks ? a.sinks[head] * LOG2E : 0.0f) - m) : 0.0f;
+}
+
 // ---------------------------------------------------------------- 32-bit, any shape
 IT_DEV float block_max(float v, float* red) {
     v = group_max<64>(v);
@@ -70,7 +77,7 @@ __global__ __launch_bounds__(256) void attend_bias_plain_k(BiasAttnP a, float* _
     for (int i = tid; i < a.v_dim; i += 256) os[i] = 0.0f;
     __syncthreads();
     float m = -INFINITY, l = 0.0f;
-    for (int s0 = 0; s0 <= pos; s0 += 256) {
+    for (int s0 = first_seen(a, pos); s0 <= pos; s0 += 256) {
         const int s = s0 + tid, live = min(256, pos + 1 - s0);
         float sc = -INFINITY;
         if (s <= pos) {
@@ -87,14 +94,14 @@ __global__ __launch_bounds__(256) void attend_bias_plain_k(BiasAttnP a, float* _
         m = m_new;
         for (int i = tid; i < a.v_dim; i += 256) {
             float acc = os[i] * alpha;
-            const int64_t at = s0 * vrow + (int64_t)kvh * a.v_stride + i;
+            const int64_t at = (int64_t)s0 * vrow + (int64_t)kvh * a.v_stride + i;
             for (int c = 0; c < live; c++)
                 acc = fmaf(ps[c], F32 ? ((const float*)a.v)[at + c * vrow] : it_f16_to_f32(((const uint16_t*)a.v)[at + c * vrow]), acc);
             os[i] = acc;
         }
         __syncthreads();
     }
-    const float den = l + (a.sink ? expf(-m) : 0.0f);
+    const float den = l + (a.sink ? expf((a.sinks ? a.sinks[h] : 0.0f) - m) : 0.0f);
     for (int i = tid; i < a.v_dim; i += 256) out[((int64_t)t * a.n_head + h) * a.v_dim + i] = os[i] / den;
 }
 
@@ -164,10 +171,10 @@ template <int HD> struct KvTile {
 struct Softmax {
     float m = -INFINITY, l = 0.0f;
     // sc: raw products (already times scale * log2 e); key of (kk, i) = key0 + 32 kk + 8 (i / 4) + 4 g + i % 4; keys past
-    // `last` are not seen; returns the factor of what was accumulated so far
-    // MASKED: some key of the tile lies past `last`
+    // `last` or ahead of `first` are not seen; returns the factor of what was accumulated so far
+    // MASKED: some key of the tile lies past `last` or ahead of `first`
     template <bool MASKED>
-    IT_DEV float step(v16f (&sc)[2], int key0, int g, int last, float pos, float slope2, h8 (&ph)[4], h8 (&pl)[4]) {
+    IT_DEV float step(v16f (&sc)[2], int key0, int g, int first, int last, float pos, float slope2, h8 (&ph)[4], h8 (&pl)[4]) {
         const float at = -slope2 * (pos - (float)(key0 + 4 * g));   // the bias of the lane's first key; the others are whole steps on
         float mt = -INFINITY;
 #pragma unroll
@@ -176,7 +183,7 @@ struct Softmax {
             for (int i = 0; i < 16; i++) {
                 const int off = 32 * kk + 8 * (i >> 2) + (i & 3);
                 float v = sc[kk][i] + fmaf(slope2, (float)off, at);
-                if (MASKED) v = key0 + 4 * g + off <= last ? v : -INFINITY;
+                if (MASKED) v = key0 + 4 * g + off <= last && key0 + 4 * g + off >= first ? v : -INFINITY;
                 sc[kk][i] = v;
                 mt = fmaxf(mt, v);
             }
@@ -224,8 +231,8 @@ __global__ __launch_bounds__(256) void attend_bias_split_k(BiasAttnP a, int n_sp
     const int h0 = kvh * G + first, split = blockIdx.y;
     const int n_pos_last = a.n_pos_dyn ? *a.n_pos_dyn : a.n_pos;
     const int pos = n_pos_last - a.n_q + t, n_pos = pos + 1;
-    const int kpb = max(16, ((n_pos + n_split - 1) / n_split + 15) & ~15);
-    const int k0 = split * kpb, k1 = min(n_pos, k0 + kpb);
+    const int seen = first_seen(a, pos), kpb = max(16, ((n_pos - seen + n_split - 1) / n_split + 15) & ~15);
+    const int k0 = seen + split * kpb, k1 = min(n_pos, k0 + kpb);
     const int64_t head_stride = (int64_t)n_split * (HD + 2);
     float* my = part + (((int64_t)t * a.n_head + h0) * n_split + split) * (HD + 2);
     if (k0 >= k1) {
@@ -274,8 +281,8 @@ __global__ __launch_bounds__(256) void attend_bias_split_k(BiasAttnP a, int n_sp
                 sc[kk] = __builtin_amdgcn_mfma_f32_32x32x16_f16(*(const h8*)(Ks + (32 * kk + c) * KS + 16 * s + 8 * g), qf, sc[kk], 0, 0, 0);
         }
         h8 ph[4], pl[4];
-        const float alpha = key0 + KT <= k1 ? sm.step<false>(sc, key0, g, k1 - 1, (float)pos, slope2, ph, pl)
-                                            : sm.step<true>(sc, key0, g, k1 - 1, (float)pos, slope2, ph, pl);
+        const float alpha = key0 + KT <= k1 ? sm.step<false>(sc, key0, g, k0, k1 - 1, (float)pos, slope2, ph, pl)
+                                            : sm.step<true>(sc, key0, g, k0, k1 - 1, (float)pos, slope2, ph, pl);
         if (kt > 0) {
 #pragma unroll
             for (int dw = 0; dw < NDW; dw++)
@@ -322,8 +329,7 @@ __global__ __launch_bounds__(256) void attend_bias_split_k(BiasAttnP a, int n_sp
 
 // one block per (query, head, 32 output dims): the weights of up to 256 splits in LDS, eight groups of 32 threads over them
 constexpr int SPLIT_MAX = 256;
-__global__ __launch_bounds__(256) void attend_bias_merge_k(const float* __restrict__ part, int n_split, int hd, int v_dim, int sink,
-                                                           float* __restrict__ out) {
+__global__ __launch_bounds__(256) void attend_bias_merge_k(BiasAttnP a, const float* __restrict__ part, int n_split, int hd, float* __restrict__ out) {
     __shared__ float wsplit[SPLIT_MAX], red[4], accs[8][32];
     const int tid = threadIdx.x, sg = tid >> 5, i = tid & 31, d = blockIdx.y * 32 + i;
     const float* p = part + (int64_t)blockIdx.x * n_split * (hd + 2);
@@ -339,7 +345,7 @@ __global__ __launch_bounds__(256) void attend_bias_merge_k(const float* __restri
     const float m = block_max(ms, red);
     const float wgt = ms != -INFINITY ? __builtin_amdgcn_exp2f(ms - m) : 0.0f;
     wsplit[tid] = wgt;
-    const float l = block_total(ls * wgt, red) + (sink ? __builtin_amdgcn_exp2f(-m) : 0.0f);
+    const float l = block_total(ls * wgt, red) + sink_share(a, blockIdx.x % a.n_head, m);
     float acc = 0.0f;
 #pragma unroll
     for (int j = 0; j < SPLIT_MAX / 8; j++) {
@@ -348,9 +354,9 @@ __global__ __launch_bounds__(256) void attend_bias_merge_k(const float* __restri
     }
     accs[sg][i] = acc;
     __syncthreads();
-    if (tid < 32 && d < v_dim) {
+    if (tid < 32 && d < a.v_dim) {
         const float r = ((accs[0][i] + accs[1][i]) + (accs[2][i] + accs[3][i])) + ((accs[4][i] + accs[5][i]) + (accs[6][i] + accs[7][i]));
-        out[(int64_t)blockIdx.x * v_dim + d] = r / l;
+        out[(int64_t)blockIdx.x * a.v_dim + d] = r / l;
     }
 }
 
@@ -393,7 +399,8 @@ __global__ __launch_bounds__(256) void attend_bias_batch_k(BiasAttnP a, int chun
         *(uint2*)(Qs + qr * KS + d) = make_uint2(lo, hi);
     }
     const int first_pos = base_pos + qt * QT, last_pos = base_pos + min(a.n_q, (qt + 1) * QT) - 1;
-    const int n_kt = last_pos / KT + 1;
+    const int n_kt = last_pos / KT + 1, kt0 = first_seen(a, first_pos) / KT, seen_by_all = first_seen(a, last_pos);
+    const int seen = first_seen(a, pos);
     Tile tile(a, kvh);
     v16f o[ND];
 #pragma unroll
@@ -401,9 +408,9 @@ __global__ __launch_bounds__(256) void attend_bias_batch_k(BiasAttnP a, int chun
 #pragma unroll
         for (int i = 0; i < 16; i++) o[dt][i] = 0.0f;
     Softmax sm;
-    tile.fetch_k(0, a.n_pos);
-    tile.fetch_v(0, a.n_pos);
-    for (int kt = 0; kt < n_kt; kt++) {
+    tile.fetch_k(kt0 * KT, a.n_pos);
+    tile.fetch_v(kt0 * KT, a.n_pos);
+    for (int kt = kt0; kt < n_kt; kt++) {
         tile.stash_k(Ks);
         tile.stash_v(Vt);
         __syncthreads();
@@ -425,8 +432,9 @@ __global__ __launch_bounds__(256) void attend_bias_batch_k(BiasAttnP a, int chun
             if ((s & 3) == 3) __builtin_amdgcn_sched_barrier(0);   // a few fragments in flight: registers are short
         }
         h8 ph[4], pl[4];
-        const float alpha = kt * KT + KT - 1 <= first_pos ? sm.step<false>(sc, kt * KT, g, pos, (float)pos, slope2, ph, pl)
-                                                          : sm.step<true>(sc, kt * KT, g, pos, (float)pos, slope2, ph, pl);
+        const float alpha = kt * KT + KT - 1 <= first_pos && kt * KT >= seen_by_all
+                                ? sm.step<false>(sc, kt * KT, g, seen, pos, (float)pos, slope2, ph, pl)
+                                : sm.step<true>(sc, kt * KT, g, seen, pos, (float)pos, slope2, ph, pl);
         if (__any(alpha != 1.0f)) {
 #pragma unroll
             for (int dt = 0; dt < ND; dt++)
@@ -447,9 +455,9 @@ __global__ __launch_bounds__(256) void attend_bias_batch_k(BiasAttnP a, int chun
         }
         __syncthreads();
     }
-    const float l = sm.l + __shfl_xor(sm.l, 32, 64) + (a.sink ? __builtin_amdgcn_exp2f(-sm.m) : 0.0f);
+    const float l = sm.l + __shfl_xor(sm.l, 32, 64) + sink_share(a, head, sm.m);
     if (!valid) return;
-    const float inv = 1.0f / l;
+    const float inv = (a.gate ? sigmoid_exact(a.gate[(int64_t)token * a.n_head + head]) : 1.0f) / l;
     const int width = a.n_head * a.v_dim;
 #pragma unroll
     for (int dt = 0; dt < ND; dt++)
@@ -522,7 +530,7 @@ size_t attend_bias_scratch_floats(const BiasAttnP& a, int n_split) {
     }
 
 bool attend_bias_split(const BiasAttnP& a, int n_split, float* scratch, float* out, hipStream_t s) {
-    if (!attend_bias_mfma_takes(a) || n_split > SPLIT_MAX) return false;
+    if (!attend_bias_mfma_takes(a) || n_split > SPLIT_MAX || !a.q || !a.k || !a.v) return false;
     const int hd = padded_head(a), G = a.n_head / a.n_head_kv, chunks = (G + 31) / 32;
     const dim3 grid((unsigned)(a.n_q * a.n_head_kv * chunks), n_split);
 #define IT_CALL(HD)                                                                                                  \
@@ -530,13 +538,12 @@ bool attend_bias_split(const BiasAttnP& a, int n_split, float* scratch, float* o
     hipLaunchKernelGGL(attend_bias_split_k<HD>, grid, dim3(256), split_lds(HD), s, a, n_split, chunks, scratch)
     IT_HEAD(hd, IT_CALL)
 #undef IT_CALL
-    hipLaunchKernelGGL(attend_bias_merge_k, dim3((unsigned)(a.n_q * a.n_head), (a.v_dim + 31) / 32), dim3(256), 0, s, scratch, n_split, hd,
-                       a.v_dim, a.sink, out);
+    hipLaunchKernelGGL(attend_bias_merge_k, dim3((unsigned)(a.n_q * a.n_head), (a.v_dim + 31) / 32), dim3(256), 0, s, a, scratch, n_split, hd, out);
     return true;
 }
 
 bool attend_bias_batch(const BiasAttnP& a, float* out32, uint16_t* out16, hipStream_t s) {
-    if (!attend_bias_mfma_takes(a) || a.n_pos_dyn) return false;
+    if (!attend_bias_mfma_takes(a) || a.n_pos_dyn || !a.q || !a.k || !a.v) return false;
     const int hd = padded_head(a), G = a.n_head / a.n_head_kv, chunks = (G + 31) / 32, cw = (G + chunks - 1) / chunks, QT = 128 / cw;
     const dim3 grid((unsigned)((a.n_q + QT - 1) / QT), (unsigned)(a.n_head_kv * chunks));
 #define IT_CALL(HD)                                                                                                  \

@@ -8,11 +8,12 @@
 // has three operands for four products) as 32 x 32 tiles of v_mfma_f32_32x32x16_bf16: lane l supplies eight k values of row l % 32 (k group l / 32)
 // for A (tokens) and B (matrix rows) and receives column l % 32 (a matrix row) and token rows
 // 8 * (i / 4) + 4 * (l / 32) + i % 4, so a store instruction writes 32 consecutive outputs of two tokens.
-// A gate / up pair shares a block: its rows are 32 gate rows, the same 32 up rows, and so on, and silu(gate) * up is
+// A gate / up pair shares a block: its rows are 32 gate rows, the same 32 up rows, and so on, and act(gate) * up is
 // formed in the lane that holds both.  A residual sum walks the terms one after the other, adds each one's scaled sums to a
 // second set of accumulators, and updates the f32 residual in place.
 #include "it_device.h"
 #include "it_float.h"
+#include "it_rows8.h"
 #include "kernels_float.h"
 
 namespace itk {
@@ -173,7 +174,7 @@ __global__ __launch_bounds__(S::THREADS, 2) void group_gemm_bf16_k(GroupP p, Til
 #pragma unroll
             for (int i = 0; i < 16; i++) {
                 const int t = t0 + 32 * mi + 8 * (i >> 2) + (i & 3);
-                if (t < p.n_tok) d.store(t, silu_exact(acc[mi][0][i]) * acc[mi][1][i]);
+                if (t < p.n_tok) d.store(t, act_of(m.act, acc[mi][0][i]) * acc[mi][1][i]);
             }
         return;
     }
@@ -244,12 +245,13 @@ __global__ __launch_bounds__(S::THREADS, 2) void res_gemm_bf16_k(ResP p, Tiles t
 #pragma unroll
             for (int ni = 0; ni < 2; ni++) {
                 const int j = j0 + 64 * wn + 32 * ni + r;
-                if (j < p.n_out) p.x[(int64_t)t * p.n_out + j] += total[mi][ni][i];
+                if (j >= p.n_out) continue;
+                float* x = p.x + (int64_t)t * p.n_out + j;
+                *x = p.set ? total[mi][ni][i] : *x + total[mi][ni][i];
             }
         }
 }
 
-bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
 template <class F> bool allow_lds(F* fn, size_t lds) {
     if (lds <= 64 * 1024) return true;
     if (hipFuncSetAttribute((const void*)fn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) == hipSuccess) return true;

@@ -3,11 +3,13 @@
 //
 // One token (decode): a launch per group.  Every block forms the normed input in LDS while its first weight rows are
 // in flight; a wave then takes groups of R rows, 16 bytes of each row a lane, and finishes them where they belong:
-// f32 rows, cache slabs, or silu(gate) * up.  Activations stay f32 throughout, so the arithmetic is the same in
+// f32 rows, cache slabs, or act(gate) * up.  What an earlier sublayer left to be normed and added to the residual is added
+// on the way in: every block forms the sum, the first one stores it, in another buffer than the one all of them read.  Activations stay f32 throughout, so the arithmetic is the same in
 // 32-bit mode.  A few tokens: one weight row a wave, eight tokens a pass.  Many tokens take k_gemm_bf16.hip.
 #include "it_device.h"
 #include "it_float.h"
 #include "it_reduce.h"
+#include "it_rows8.h"
 #include "kernels_float.h"
 
 namespace itk {
@@ -15,79 +17,11 @@ namespace {
 
 constexpr int CH = 512;   // elements of a row a wave takes at a time, eight a lane
 
-template <int FMT> struct Raw8 { uint4 a; };
-template <> struct Raw8<W_F32> { uint4 a, b; };
-
-template <int FMT> IT_DEV const uint8_t* row_at(const uint8_t* w, int64_t row, int n_in) {
-    return w + row * n_in * (FMT == W_F32 ? 4 : 2);
-}
-// a weight is read once a token: it need not stay in the caches
-typedef uint32_t u4 __attribute__((ext_vector_type(4)));
-IT_DEV uint4 stream16(const void* p) {
-    const u4 v = __builtin_nontemporal_load((const u4*)p);
-    return make_uint4(v.x, v.y, v.z, v.w);
-}
-// eight elements of a row from k on; AL: the row length is a multiple of 8 and the rows are 16-byte aligned
-template <int FMT, bool AL> IT_DEV Raw8<FMT> load8(const uint8_t* row, int k, int n_in) {
-    Raw8<FMT> r{};
-    if (AL) {
-        if (k < n_in) {
-            if constexpr (FMT == W_F32) {
-                r.a = stream16((const float*)row + k);
-                r.b = stream16((const float*)row + k + 4);
-            } else {
-                r.a = stream16((const uint16_t*)row + k);
-            }
-        }
-    } else {
-        uint32_t v[8];
-#pragma unroll
-        for (int e = 0; e < 8; e++) {
-            if (FMT == W_F32) v[e] = k + e < n_in ? ((const uint32_t*)row)[k + e] : 0u;
-            else v[e] = k + e < n_in ? ((const uint16_t*)row)[k + e] : 0u;
-        }
-        if constexpr (FMT == W_F32) {
-            r.a = make_uint4(v[0], v[1], v[2], v[3]);
-            r.b = make_uint4(v[4], v[5], v[6], v[7]);
-        } else {
-            r.a = make_uint4(v[0] | (v[1] << 16), v[2] | (v[3] << 16), v[4] | (v[5] << 16), v[6] | (v[7] << 16));
-        }
-    }
-    return r;
-}
-template <int FMT> IT_DEV void widen8(const Raw8<FMT>& r, float* f) {
-    if constexpr (FMT == W_F32) {
-        const uint32_t v[8] = {r.a.x, r.a.y, r.a.z, r.a.w, r.b.x, r.b.y, r.b.z, r.b.w};
-#pragma unroll
-        for (int e = 0; e < 8; e++) f[e] = __uint_as_float(v[e]);
-    } else {
-        const uint32_t v[4] = {r.a.x, r.a.y, r.a.z, r.a.w};
-#pragma unroll
-        for (int e = 0; e < 4; e++) {
-            if (FMT == W_BF16) {
-                f[2 * e] = __uint_as_float(v[e] << 16);
-                f[2 * e + 1] = __uint_as_float(v[e] & 0xffff0000u);
-            } else {
-                f[2 * e] = it_f16_to_f32((uint16_t)(v[e] & 0xffffu));
-                f[2 * e + 1] = it_f16_to_f32((uint16_t)(v[e] >> 16));
-            }
-        }
-    }
-}
-
 // which matrix a group of rows belongs to
 struct Groups {
     int first[GROUP_MAX + 1];
     int n;
 };
-
-IT_DEV float block_sum(float v, float* red) {   // 256 threads
-    v = group_sum<64>(v);
-    __syncthreads();
-    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
-    __syncthreads();
-    return (red[0] + red[1]) + (red[2] + red[3]);
-}
 
 constexpr int U = 4;   // row pieces of a wave in flight
 
@@ -129,7 +63,33 @@ __global__ __launch_bounds__(256) void group_gemv_k(GroupP p, Groups gs) {
     // the input while the first rows are on their way
     {
         float ss = 0.0f;
-        if (p.n_in % 4 == 0) {   // (device buffers are 16-byte aligned)
+        if (p.add.y) {
+            float *x0 = xs + n_ch * CH, sy = 0.0f;   // the residual behind the input
+            if (p.n_in % 4 == 0) {
+                for (int i = tid * 4; i < p.n_in; i += 1024) {
+                    const float4 v = *(const float4*)(p.add.y + i);
+                    *(float4*)(x0 + i) = *(const float4*)(p.x + i);
+                    sy = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, sy))));
+                    *(float4*)(xs + i) = v;
+                }
+                for (int i = p.n_in + tid * 4; i < n_ch * CH; i += 1024) *(float4*)(xs + i) = make_float4(0.f, 0.f, 0.f, 0.f);
+            } else {
+                for (int i = tid; i < n_ch * CH; i += 256) {
+                    const float v = i < p.n_in ? p.add.y[i] : 0.0f;
+                    if (i < p.n_in) x0[i] = p.x[i];
+                    sy = fmaf(v, v, sy);
+                    xs[i] = v;
+                }
+            }
+            sy = block_sum(sy, red);   // (its barriers also publish xs and x0)
+            const float r = p.add.mult / sqrtf(sy / (float)p.n_in + p.add.eps);
+            for (int i = tid; i < p.n_in; i += 256) {
+                const float v = fmaf(xs[i] * p.add.w[i], r, x0[i]);
+                ss = fmaf(v, v, ss);
+                xs[i] = v;
+                if (blockIdx.x == 0) p.add.x_new[i] = v;
+            }
+        } else if (p.n_in % 4 == 0) {   // (device buffers are 16-byte aligned)
             for (int i = tid * 4; i < n_ch * CH; i += 1024) {
                 const float4 v = i < p.n_in ? *(const float4*)(p.x + i) : make_float4(0.f, 0.f, 0.f, 0.f);
                 ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
@@ -178,7 +138,7 @@ __global__ __launch_bounds__(256) void group_gemv_k(GroupP p, Groups gs) {
         if (m.up) {
 #pragma unroll
             for (int r = 0; r < R / 2; r++)
-                if (lane == r && j0 + r < m.n_out) group_store(m, 0, j0 + r, silu_exact(acc[r]) * acc[R / 2 + r]);
+                if (lane == r && j0 + r < m.n_out) group_store(m, 0, j0 + r, act_of(m.act, acc[r]) * acc[R / 2 + r]);
         } else {
 #pragma unroll
             for (int r = 0; r < R; r++)
@@ -250,7 +210,10 @@ __global__ __launch_bounds__(512) void res_gemv_k(ResP p) {
                 }
                 const float rinv = 1.0f / sqrtf(ss / (float)part + t.eps);
                 if (gi < t.norm_groups)
-                    for (int i = sub * 64 + lane; i < part; i += 64 * wpg) a[i] = a[i] * rinv * t.norm_w[gi * part + i];
+                    for (int i = sub * 64 + lane; i < part; i += 64 * wpg) {
+                        const float v = a[i] * rinv * t.norm_w[t.norm_period == part ? i : gi * part + i];
+                        a[i] = t.gate ? v * silu_exact(t.gate[gi * part + i]) : v;
+                    }
             }
         }
         at += (t.n_in + CH - 1) / CH * CH;
@@ -301,7 +264,7 @@ __global__ __launch_bounds__(512) void res_gemv_k(ResP p) {
             }
             total += p.t[k].scale ? v * p.t[k].scale[j0 + r] : v;
         }
-        p.x[j0 + r] += total;
+        p.x[j0 + r] = p.set ? total : p.x[j0 + r] + total;
     }
 }
 
@@ -342,7 +305,7 @@ __global__ __launch_bounds__(256) void group_rows_k(GroupP p, Groups gs) {   // 
     if (m.up) dot_rows<FMT, AL>(row_at<FMT>(m.up, j, p.n_in), p.x, p.n_in, p.n_tok, t0, lane, b);
 #pragma unroll
     for (int t = 0; t < NT; t++)
-        if (lane == t && t0 + t < p.n_tok) group_store(m, t0 + t, j, m.up ? silu_exact(a[t]) * b[t] : a[t]);
+        if (lane == t && t0 + t < p.n_tok) group_store(m, t0 + t, j, m.up ? act_of(m.act, a[t]) * b[t] : a[t]);
 }
 
 template <int FMT, bool AL>
@@ -362,7 +325,10 @@ __global__ __launch_bounds__(256) void res_rows_k(ResP p) {
     }
 #pragma unroll
     for (int t = 0; t < NT; t++)
-        if (lane == t && t0 + t < p.n_tok) p.x[(int64_t)(t0 + t) * p.n_out + j] += total[t];
+        if (lane == t && t0 + t < p.n_tok) {
+            float* x = p.x + (int64_t)(t0 + t) * p.n_out + j;
+            *x = p.set ? total[t] : *x + total[t];
+        }
 }
 
 // ---------------------------------------------------------------- norms, conversions, sums
@@ -419,6 +385,93 @@ __global__ __launch_bounds__(256) void norm_rows4_k(const float* __restrict__ x,
     }
 }
 
+// a wave a part (a head's output, as a rule)
+__global__ __launch_bounds__(256) void norm_gate_rows_k(const float* __restrict__ x, const float* __restrict__ w, int period, const float* __restrict__ gate,
+                                                        int groups, float eps, int64_t n_parts, int nd, float* __restrict__ out32, uint16_t* __restrict__ out16) {
+    const int part = nd / groups, lane = threadIdx.x & 63;
+    const int64_t at = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (at >= n_parts) return;
+    const int64_t row = at / groups;
+    const int j0 = (int)(at % groups) * part;
+    const float* xr = x + row * nd + j0;
+    float ss = 0.0f;
+    for (int i = lane; i < part; i += 64) ss = fmaf(xr[i], xr[i], ss);
+    const float rinv = 1.0f / sqrtf(group_sum<64>(ss) / (float)part + eps);
+    for (int i = lane; i < part; i += 64) {
+        float v = xr[i] * rinv * w[period == part ? i : j0 + i];
+        if (gate) v *= silu_exact(gate[row * nd + j0 + i]);
+        if (out32) out32[row * nd + j0 + i] = v;
+        if (out16) out16[row * pad8(nd) + j0 + i] = to_bf16(v);
+    }
+    if (out16 && j0 + part == nd && lane < pad8(nd) - nd) out16[row * pad8(nd) + nd + lane] = 0;
+}
+
+// V > 0: rows of whole float4s, a thread keeps its V pieces; V = 0: any row, through x_new
+template <int V>
+__global__ __launch_bounds__(256) void add_norm_rows_k(const float* __restrict__ x, AddNormed a, const float* __restrict__ w, float eps, int nd,
+                                                       float* __restrict__ out32, uint16_t* __restrict__ out16) {
+    __shared__ float red[4];
+    const int tid = threadIdx.x;
+    const int64_t row = blockIdx.x;
+    const float *xr = x + row * nd, *yr = a.y + row * nd;
+    float *xn = a.x_new + row * nd, sy = 0.0f, ss = 0.0f;
+    if constexpr (V > 0) {
+        const int n4 = nd >> 2;
+        float4 xv[V], yv[V];
+#pragma unroll
+        for (int i = 0; i < V; i++) {
+            const int at = tid + i * 256;
+            xv[i] = at < n4 ? ((const float4*)xr)[at] : make_float4(0.f, 0.f, 0.f, 0.f);
+            yv[i] = at < n4 ? ((const float4*)yr)[at] : make_float4(0.f, 0.f, 0.f, 0.f);
+            sy = fmaf(yv[i].x, yv[i].x, fmaf(yv[i].y, yv[i].y, fmaf(yv[i].z, yv[i].z, fmaf(yv[i].w, yv[i].w, sy))));
+        }
+        const float r = a.mult / sqrtf(block_sum(sy, red) / (float)nd + a.eps);
+#pragma unroll
+        for (int i = 0; i < V; i++) {
+            const int at = tid + i * 256;
+            if (at >= n4) continue;
+            const float4 ww = ((const float4*)a.w)[at];
+            float4& v = xv[i];
+            v = make_float4(fmaf(yv[i].x * ww.x, r, v.x), fmaf(yv[i].y * ww.y, r, v.y), fmaf(yv[i].z * ww.z, r, v.z), fmaf(yv[i].w * ww.w, r, v.w));
+            ((float4*)xn)[at] = v;
+            ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+        }
+        if (!w) return;
+        const float rinv = 1.0f / sqrtf(block_sum(ss, red) / (float)nd + eps);
+#pragma unroll
+        for (int i = 0; i < V; i++) {
+            const int at = tid + i * 256;
+            if (at >= n4) continue;
+            const float4 ww = ((const float4*)w)[at], v = xv[i];
+            const float4 h = make_float4(v.x * rinv * ww.x, v.y * rinv * ww.y, v.z * rinv * ww.z, v.w * rinv * ww.w);
+            if (out32) ((float4*)(out32 + row * nd))[at] = h;
+            if (out16)
+                ((uint2*)(out16 + row * nd))[at] = make_uint2(to_bf16(h.x) | ((uint32_t)to_bf16(h.y) << 16), to_bf16(h.z) | ((uint32_t)to_bf16(h.w) << 16));
+        }
+    } else {
+        for (int i = tid; i < nd; i += 256) sy = fmaf(yr[i], yr[i], sy);
+        const float r = a.mult / sqrtf(block_sum(sy, red) / (float)nd + a.eps);
+        for (int i = tid; i < nd; i += 256) {
+            const float v = fmaf(yr[i] * a.w[i], r, xr[i]);
+            xn[i] = v;
+            ss = fmaf(v, v, ss);
+        }
+        if (!w) return;
+        const float rinv = 1.0f / sqrtf(block_sum(ss, red) / (float)nd + eps);
+        for (int i = tid; i < nd; i += 256) {   // (a thread's own elements)
+            const float h = xn[i] * rinv * w[i];
+            if (out32) out32[row * nd + i] = h;
+            if (out16) out16[row * pad8(nd) + i] = to_bf16(h);
+        }
+        if (out16 && tid < pad8(nd) - nd) out16[row * pad8(nd) + nd + tid] = 0;
+    }
+}
+
+__global__ void act_mul_k(float* __restrict__ a, const float* __restrict__ b, int64_t n, int act) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i < n) a[i] = act_of(act, a[i]) * b[i];
+}
+
 __global__ void widen_rows_k(const uint16_t* __restrict__ in, int nd, float* __restrict__ out, int64_t n) {
     const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (i < n) out[i] = it_bf16_to_f32(in[i / nd * pad8(nd) + i % nd]);
@@ -431,13 +484,13 @@ __global__ void group_scatter_k(GroupMat m, const float* __restrict__ rows, int6
 }
 
 __global__ void scaled_residual_k(float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ sa,
-                                  const float* __restrict__ b, const float* __restrict__ sb, int nd, int64_t n) {
+                                  const float* __restrict__ b, const float* __restrict__ sb, int set, int nd, int64_t n) {
     const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (i >= n) return;
     const int j = (int)(i % nd);
     float v = sa ? a[i] * sa[j] : a[i];
     if (b) v += sb ? b[i] * sb[j] : b[i];
-    x[i] += v;
+    x[i] = set ? v : x[i] + v;
 }
 
 __global__ void add_rows_k(float* __restrict__ x, const float* __restrict__ rows, const float* __restrict__ vec, int nd, int64_t n) {
@@ -454,8 +507,6 @@ __global__ void gather_rows_k(const float* __restrict__ src, const int32_t* __re
     if (i >= n) return;
     out[i] = src[(int64_t)idx[i / nd] * nd + i % nd];
 }
-
-bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
 
 Groups groups_of(const GroupP& p, int rows_per_group) {
     Groups g{};
@@ -477,6 +528,7 @@ bool res_aligned(const ResP& p) {
     return al;
 }
 size_t padded(int n) { return (size_t)((n + CH - 1) / CH * CH); }
+size_t group_lds(const GroupP& p) { return padded(p.n_in) * (p.add.y ? 2 : 1) * sizeof(float); }
 constexpr size_t LDS_MAX = 144 * 1024;
 
 template <class F> bool allow_lds(F* fn, size_t lds) {
@@ -487,7 +539,7 @@ template <class F> bool allow_lds(F* fn, size_t lds) {
 }
 
 template <int FMT, bool AL> bool launch_group(const GroupP& p, hipStream_t s) {
-    const size_t lds = padded(p.n_in) * sizeof(float);
+    const size_t lds = group_lds(p);
     Groups g4 = groups_of(p, 4);
     if (g4.n >= 2048) {   // enough groups of four rows to keep every wave of the chip at work
         if (!allow_lds(group_gemv_k<FMT, AL, 4>, lds)) return false;
@@ -518,17 +570,9 @@ template <int FMT, bool AL> bool launch_res(const ResP& p, hipStream_t s) {
 #undef IT_RES
 }
 
-// one call per (format, alignment)
-#define IT_BY_FORMAT(fmt, al, CALL)                                                    \
-    do {                                                                               \
-        if ((fmt) == W_BF16) { if (al) { CALL(W_BF16, true); } else { CALL(W_BF16, false); } } \
-        else if ((fmt) == W_F16) { if (al) { CALL(W_F16, true); } else { CALL(W_F16, false); } } \
-        else { if (al) { CALL(W_F32, true); } else { CALL(W_F32, false); } }           \
-    } while (0)
-
 }  // namespace
 
-bool group_gemv_takes(const GroupP& p) { return p.n_tok == 1 && padded(p.n_in) * sizeof(float) <= LDS_MAX; }
+bool group_gemv_takes(const GroupP& p) { return p.n_tok == 1 && group_lds(p) <= LDS_MAX; }
 bool group_gemv(const GroupP& p, hipStream_t s) {
     if (!group_gemv_takes(p)) return false;
     const bool al = group_aligned(p);
@@ -584,6 +628,28 @@ void norm_rows(const float* x, const float* w, int groups, float eps, int64_t n_
     hipLaunchKernelGGL(norm_rows_k, dim3((unsigned)n_rows, groups), dim3(256), 0, s, x, w, groups, eps, nd, out32, out16);
 }
 
+void norm_gate_rows(const float* x, const float* w, int period, const float* gate, int groups, float eps, int64_t n_rows, int nd,
+                    float* out32, uint16_t* out16, hipStream_t s) {
+    if (n_rows <= 0) return;
+    const int64_t parts = n_rows * groups;
+    hipLaunchKernelGGL(norm_gate_rows_k, dim3((unsigned)((parts + 3) / 4)), dim3(256), 0, s, x, w, period, gate, groups, eps, parts, nd, out32, out16);
+}
+
+void add_norm_rows(const float* x, const AddNormed& add, const float* norm_w, float eps, int64_t n_rows, int nd, float* out32,
+                   uint16_t* out16, hipStream_t s) {
+    if (n_rows <= 0) return;
+    const dim3 grid((unsigned)n_rows), block(256);
+    const bool al = nd % 8 == 0 && aligned16(x) && aligned16(add.y) && aligned16(add.x_new) && aligned16(add.w) && aligned16(norm_w) &&
+                    aligned16(out32) && aligned16(out16);
+#define IT_CALL(V) hipLaunchKernelGGL(add_norm_rows_k<V>, grid, block, 0, s, x, add, norm_w, eps, nd, out32, out16)
+    if (!al || nd > 8192) IT_CALL(0);
+    else if (nd <= 1024) IT_CALL(1);
+    else if (nd <= 2048) IT_CALL(2);
+    else if (nd <= 4096) IT_CALL(4);
+    else IT_CALL(8);
+#undef IT_CALL
+}
+
 static dim3 per_element(int64_t n) { return dim3((unsigned)((n + 255) / 256)); }
 void widen_rows(const uint16_t* in, int64_t n_rows, int nd, float* out, hipStream_t s) {
     const int64_t n = n_rows * nd;
@@ -593,9 +659,12 @@ void group_scatter(const GroupMat& m, const float* rows, int n_tok, hipStream_t 
     const int64_t n = (int64_t)n_tok * m.n_out;
     hipLaunchKernelGGL(group_scatter_k, per_element(n), dim3(256), 0, s, m, rows, n);
 }
-void scaled_residual(float* x, const float* a, const float* sa, const float* b, const float* sb, int64_t n_rows, int nd, hipStream_t s) {
+void scaled_residual(float* x, const float* a, const float* sa, const float* b, const float* sb, int set, int64_t n_rows, int nd, hipStream_t s) {
     const int64_t n = n_rows * nd;
-    hipLaunchKernelGGL(scaled_residual_k, per_element(n), dim3(256), 0, s, x, a, sa, b, sb, nd, n);
+    hipLaunchKernelGGL(scaled_residual_k, per_element(n), dim3(256), 0, s, x, a, sa, b, sb, set, nd, n);
+}
+void act_mul(float* a, const float* b, int64_t n, int act, hipStream_t s) {
+    hipLaunchKernelGGL(act_mul_k, per_element(n), dim3(256), 0, s, a, b, n, act);
 }
 void add_rows(float* x, const float* rows, const float* vec, int64_t n_rows, int nd, hipStream_t s) {
     const int64_t n = n_rows * nd;

@@ -19,13 +19,13 @@
 
 #include "it_device.h"
 #include "it_float.h"
+#include "it_mfma32.h"
 #include "it_reduce.h"
 #include "kernels_float.h"
 
 namespace itk {
 namespace {
 
-typedef float v4f __attribute__((ext_vector_type(4)));
 constexpr int PR = 16;     // value rows per block
 constexpr int TAPS_MAX = 16;
 constexpr int N_MAX = 512;
@@ -201,21 +201,6 @@ __global__ __launch_bounds__(256) void ssd_scan_k(SsdP p) {
 constexpr int L = 64;
 constexpr int PW = 64;      // value rows of a head per block
 constexpr int XS = PW + 4;  // LDS row stride of the inputs
-// D = A(16 x 4) B(4 x 16) + C: lane l gives A[l % 16][l / 16] and B[l / 16][l % 16], and holds D[4 * (l / 16) + i][l % 16].
-// The order of k is free as long as both operands agree: four products in turn take k = 4 (l / 16) + 0 .. 3 of a stretch of
-// 16, so that a lane's operands are 16 bytes in a row.
-IT_DEV v4f mfma4(float a, float b, v4f c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
-IT_DEV v4f mfma16(const float4& a, const float4& b, v4f c) {
-    c = mfma4(a.x, b.x, c);
-    c = mfma4(a.y, b.y, c);
-    c = mfma4(a.z, b.z, c);
-    return mfma4(a.w, b.w, c);
-}
-// four elements of a row of n from k on, zeros past its end
-IT_DEV float4 row4(const float* q, int k, int n, bool vec) {
-    if (vec) return k < n ? *(const float4*)(q + k) : make_float4(0.f, 0.f, 0.f, 0.f);
-    return make_float4(k < n ? q[k] : 0.0f, k + 1 < n ? q[k + 1] : 0.0f, k + 2 < n ? q[k + 2] : 0.0f, k + 3 < n ? q[k + 3] : 0.0f);
-}
 IT_DEV bool rows_vec(const SsdP& p) { return p.n % 4 == 0 && p.inner() % 4 == 0; }
 
 // a call's chunks are taken a stretch at a time (ck0 ..): per stretch

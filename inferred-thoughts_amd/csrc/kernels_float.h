@@ -26,32 +26,45 @@ struct GroupOut {
 };
 struct GroupMat {
     const uint8_t* w;
-    const uint8_t* up;          // non-null: the result is silu(w x) * (up x)
+    const uint8_t* up;          // non-null: the result is act(w x) * (up x)
     int n_out;
+    int act;                    // ACT_*
     float scale;
     GroupOut o;
 };
+enum { ACT_SILU = 0, ACT_RELU = 1 };
+// x_new = x + mult * (y / rms(y)) * w: what a sublayer whose output is normed adds to the residual
+struct AddNormed {
+    const float* y;             // [token][n], or null: nothing to add
+    const float* w;             // [n]
+    float* x_new;               // [token][n], another buffer than x
+    float eps, mult;
+};
 struct GroupP {
     const float* x;             // [token][n_in]
+    AddNormed add;              // what is added to x ahead of the norm
     const float* norm_w;        // RMS norm ahead of the products, or null
     float eps;
     int n_in, n_tok, n_mats, fmt;
     GroupMat m[GROUP_MAX];
 };
 
-// x[t][j] += sum over the terms of scale[j] * (W norm(in))[j]
+// x[t][j] += (set: =) sum over the terms of scale[j] * (W norm(in))[j]
 struct ResTerm {
     const uint8_t* w;
     const float* in;            // [token][n_in]
     const float* scale;         // [n_out] or null
     const float* norm_w;        // RMS norm of `norm_groups` equal parts ahead of the product, or null
+    const float* gate;          // [token][n_in]: the normed input times silu(gate), or null
     int n_in, norm_groups;
+    int norm_period;            // elements of norm_w, used again and again along the row: n_in, or a part
     float eps;
 };
 constexpr int RES_MAX = 2;
 struct ResP {
     float* x;
     int n_out, n_tok, n_terms, fmt;
+    int set;
     ResTerm t[RES_MAX];
 };
 
@@ -72,12 +85,20 @@ void res_gemm_bf16(const ResP& p, const uint16_t* const in16[RES_MAX], hipStream
 // to f32 and / or to bf16 rows of pad8(nd)
 void norm_rows(const float* x, const float* w, int groups, float eps, int64_t n_rows, int nd, float* out32, uint16_t* out16,
                hipStream_t s);
+// the same with w of `period` elements repeated along the row, and silu(gate) behind it
+void norm_gate_rows(const float* x, const float* w, int period, const float* gate, int groups, float eps, int64_t n_rows, int nd,
+                    float* out32, uint16_t* out16, hipStream_t s);
+// x_new = x + what `add` says; with norm_w also rms(x_new) * norm_w to f32 and / or to bf16 rows of pad8(nd)
+void add_norm_rows(const float* x, const AddNormed& add, const float* norm_w, float eps, int64_t n_rows, int nd, float* out32,
+                   uint16_t* out16, hipStream_t s);
+// a = act(a) * b
+void act_mul(float* a, const float* b, int64_t n, int act, hipStream_t s);
 // f32 rows of nd from bf16 rows of pad8(nd)
 void widen_rows(const uint16_t* in, int64_t n_rows, int nd, float* out, hipStream_t s);
 // one matrix's f32 rows to where its GroupOut says (the form with one launch per operation)
 void group_scatter(const GroupMat& m, const float* rows, int n_tok, hipStream_t s);
 // x += a * sa (+ b * sb), the sum of the two first; scales [nd] or null, b may be null
-void scaled_residual(float* x, const float* a, const float* sa, const float* b, const float* sb, int64_t n_rows, int nd, hipStream_t s);
+void scaled_residual(float* x, const float* a, const float* sa, const float* b, const float* sb, int set, int64_t n_rows, int nd, hipStream_t s);
 // x[t] += rows[t] (may be null) + 1 * vec: the row first, then the vector (may be null)
 void add_rows(float* x, const float* rows, const float* vec, int64_t n_rows, int nd, hipStream_t s);
 void gather_rows(const float* src, const int32_t* idx, int n_rows, int nd, float* out, hipStream_t s);
@@ -91,7 +112,10 @@ struct BiasAttnP {
     int k_dim, v_dim, k_stride, v_stride, n_head, n_head_kv;
     float scale;
     const float* slopes;        // [n_head] (device) or null: score -= slope * (i - j)
-    int sink;                   // 1: the denominator is 1 + sum exp(score)
+    int sink;                   // 1: the denominator is e^sinks[head] + sum exp(score)
+    const float* sinks;         // [n_head] (device) or null: all 0
+    int window;                 // position i sees the keys above i - window; 0: all up to i
+    const float* gate;          // [token][n_head]: the output times sigmoid(gate), or null (attend_bias_batch only)
     float temp_coef;            // q *= 1 + coef * ln(floor((p + 1) / every) + 1); 0: none
     int temp_every;
     const int* n_pos_dyn;
@@ -130,5 +154,63 @@ void ssd_scan(const SsdP& p, hipStream_t s);          // several tokens, one aft
 bool ssd_chunk_takes(const SsdP& p);
 size_t ssd_chunk_work_floats(const SsdP& p);
 void ssd_chunk(const SsdP& p, float* work, hipStream_t s);   // many tokens: chunks of 64 on the fp32 matrix cores
+
+
+// ---- gated linear attention: a decay per key channel ----
+struct GlaP {
+    const float *q, *k;         // [token][heads * dim]
+    const float* v;             // [token][heads * vdim]
+    const float* low;           // [token][rank]: the decay's logit is a2 low + a2_b
+    const uint8_t* a2;          // [heads * dim][rank] of type a2_fmt
+    int a2_fmt;
+    const float* a2_b;
+    float inv_tau;
+    float* state;               // [heads][vdim][dim]
+    float* decay;               // [token][heads * dim] (not used for one token): see gla_decay
+    float* out;                 // [token][heads * vdim]
+    int heads, dim, vdim, rank, n_tok;
+    __host__ __device__ int keys() const { return heads * dim; }
+    __host__ __device__ int values() const { return heads * vdim; }
+};
+bool gla_takes(const GlaP& p);
+void gla_step(const GlaP& p, hipStream_t s);          // one token
+// several tokens: the decays, or their logarithms summed up over every 16 tokens of the call
+void gla_decay(const GlaP& p, int logs, hipStream_t s);
+void gla_scan(const GlaP& p, hipStream_t s);          // several tokens, one after the other, from the decays
+bool gla_chunk_takes(const GlaP& p);
+size_t gla_chunk_work_floats(const GlaP& p);
+bool gla_chunk(const GlaP& p, float* work, hipStream_t s);   // many tokens: chunks of 64 on the fp32 matrix cores, from the logarithms
+
+// ---- latent attention: a cache row is [latent | rotated key part], shared by all heads ----
+struct LatentP {
+    const float* q;             // [token][heads * (dim + rot)]: [unrotated | rotated] a head
+    const float* kv;            // [token][rank + rot]: latent before its norm, key part before its rotation; null: rows are there already
+    const float* kv_norm;       // [rank]
+    float eps;
+    const float2* table;        // (cos, sin) of [position][n_rot / 2]
+    const uint8_t* uk;          // [heads * dim][rank] of type uk_fmt
+    const uint8_t* uv;          // [heads * vdim][rank] of type uv_fmt
+    int uk_fmt, uv_fmt;
+    void* slab;                 // row = position
+    int slab_f32, row_stride;
+    const float* gate;          // [token][heads] or null: the output times sigmoid(gate)
+    int heads, dim, rot, n_rot, rank, vdim;
+    int n_tok, pos;
+    const int* n_pos_dyn;       // one token: the context's length (position + 1)
+    __host__ __device__ int k_dim() const { return rank + rot; }
+};
+// queries against the latent itself: qa [token][heads][rank + rot] = [uk^T q | rotated q]; the tokens' cache rows
+void latent_prep(const LatentP& p, float* qa, hipStream_t s);
+// many tokens: their cache rows, and the rotated parts of q in place
+void latent_rows(const LatentP& p, float* q, hipStream_t s);
+// cache rows `first` .. as bf16 latents of pad8(rank) and as the rotated part of every head's key rows (f16, ks elements a head)
+void latent_keys(const LatentP& p, int first, int n_keys, uint16_t* c16, uint16_t* k, int ks, hipStream_t s);
+// out [token][heads * vdim] = gate * uv (merged partials of attend_shared_split; n_split 0: `part` holds [token][heads][rank])
+void latent_value(const LatentP& p, const BiasAttnP& a, const float* part, int n_split, float* out, hipStream_t s);
+// few queries against rows whose first v_dim elements are the values, one row for all heads: partial sums of f16 matrix cores
+bool attend_shared_takes(const BiasAttnP& a);
+int attend_shared_splits(const BiasAttnP& a, int n_pos_max);
+size_t attend_shared_scratch_floats(const BiasAttnP& a, int n_split);
+bool attend_shared_split(const BiasAttnP& a, int n_split, float* scratch, hipStream_t s);
 
 }  // namespace itk

@@ -28,6 +28,7 @@ struct Design {
 const Design DESIGNS[] = {
     {"qwen35moe", false, open_qwen35moe},
     {"Serisun", true, open_serisun},
+    {"Nubedra", true, open_nubedra},
 };
 
 it_model* open_model(const std::string& path, std::string* err) {
@@ -80,14 +81,19 @@ int it_engine::check_pass(const uint32_t* tokens, uint64_t n, uint64_t start) {
 int it_engine::embed(const uint32_t* tokens, uint64_t n, float* x, uint64_t ring_index) {
     const it_weights& w = model->embedding();
     const uint64_t nd = w.n_in;
+    const float scale = model->embedding_scale();
     if (tokens) {
         uint64_t row_bytes = itg::type_bytes(w.ty, nd);
         for (uint64_t t = 0; t < n; t++) ith::dequantize(w.ty, w.data + tokens[t] * row_bytes, nd, x + t * nd);
+        if (scale != 1.0f)
+            for (uint64_t i = 0; i < n * nd; i++) x[i] *= scale;
         it_hip_host_wrote(be, x, n * nd);
     } else if (!it_hip_embed_argmax(be, &w, logits.p(), model->vocab(), x, nd, ring_index)) {
         it_hip_end_pass(be);
         err = "the embedding table's type has no device form";
         return -4;
+    } else if (scale != 1.0f) {
+        it_hip_scale(be, x, nd, scale);
     }
     return 0;
 }

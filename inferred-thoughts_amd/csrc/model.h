@@ -32,6 +32,7 @@ struct it_model {
     virtual uint64_t decode_weight_bytes() const = 0;
     virtual void token_macs(uint64_t out[3]) const = 0;
     virtual const it_weights& embedding() const = 0;
+    virtual float embedding_scale() const { return 1.0f; }
     virtual it_engine* new_engine(it_hip* be, uint64_t n_ctx, uint64_t max_batch) = 0;
 
     bool fail(const std::string& m) {
@@ -75,5 +76,6 @@ struct it_engine {
 // The designs: each opens what its file format's architecture name says
 it_model* open_qwen35moe(const std::string& path, std::string* err);
 it_model* open_serisun(const std::string& dir, std::string* err);
+it_model* open_nubedra(const std::string& dir, std::string* err);
 // "architecture" of a folder's config.json
 bool config_architecture(const std::string& dir, std::string* name, std::string* err);

@@ -5,35 +5,12 @@
 //
 // A model is a folder with config.json and model.safetensors; every size and constant comes from there.
 #include <cmath>
-#include <cstdio>
 #include <cstring>
-#include <fstream>
 #include <memory>
-#include <sstream>
 
-#include "host_formats.h"
-#include "json.h"
-#include "model.h"
-#include "safetensors.h"
+#include "model_folder.h"
 
 namespace {
-
-bool read_config(const std::string& dir, itj::Value* out, std::string* err) {
-    std::ifstream f(dir + "/config.json", std::ios::binary);
-    if (!f) {
-        *err = dir + "/config.json: cannot be read";
-        return false;
-    }
-    std::stringstream s;
-    s << f.rdbuf();
-    const std::string text = s.str();
-    std::string why;
-    if (itj::parse(text.data(), text.size(), out, &why)) return true;
-    *err = dir + "/config.json: " + why;
-    return false;
-}
-
-uint64_t round8(uint64_t n) { return (n + 7) / 8 * 8; }
 
 struct Attention {
     uint64_t heads = 0, kv_heads = 0, dim = 0, vdim = 0, temp_every = 0;
@@ -67,29 +44,14 @@ struct Run {
     uint64_t slot = 0;    // of the cache's key / value slabs, or of its states
 };
 
-struct Serisun : it_model {
-    its::File file;
-    uint64_t n_vocab = 0, nd = 0, passes = 1;   // passes: through the looped layers
-    float eps = 0, logit_scale = 1;
+struct Serisun : FolderModel {
+    uint64_t passes = 1;   // through the looped layers
+    float logit_scale = 1;
     std::vector<Layer> layers;
     std::vector<Run> runs;
     std::vector<float> step, final_norm;   // step: [times][width]
-    it_weights embed_w{}, head{};
+    it_weights head{};
 
-    // ---- config.json
-    bool size(const itj::Value* o, const char* where, const char* key, uint64_t* out, uint64_t least = 1) {
-        const itj::Value* v = o ? o->get(key) : nullptr;
-        if (!v || v->kind != itj::Value::Number || v->num < (double)least || v->num > 1e9 || v->num != std::floor(v->num))
-            return fail(std::string("config.json: ") + where + "." + key + " is missing or not a whole number in range");
-        *out = (uint64_t)v->num;
-        return true;
-    }
-    bool real(const itj::Value* o, const char* where, const char* key, float* out) {
-        const itj::Value* v = o ? o->get(key) : nullptr;
-        if (!v || v->kind != itj::Value::Number) return fail(std::string("config.json: ") + where + "." + key + " is missing or not a number");
-        *out = (float)v->num;
-        return true;
-    }
     bool config(const itj::Value& c) {
         if (!size(&c, "", "vocab", &n_vocab) || !size(&c, "", "width", &nd) || !real(c.get("norm"), "norm", "eps", &eps) ||
             !real(&c, "", "logit_scale", &logit_scale))
@@ -148,35 +110,6 @@ struct Serisun : it_model {
         return !looped || vec("loop.step", {times, nd}, &step);
     }
 
-    // ---- tensors
-    const its::Tensor* need(const std::string& name, const std::vector<uint64_t>& shape) {
-        const its::Tensor* t = file.tensor(name);
-        if (!t) {
-            fail("missing tensor " + name);
-            return nullptr;
-        }
-        if (t->shape != shape) {
-            std::string m = "tensor " + name + ": expected [";
-            for (auto v : shape) m += std::to_string(v) + ",";
-            m += "] got [";
-            for (auto v : t->shape) m += std::to_string(v) + ",";
-            fail(m + "]");
-            return nullptr;
-        }
-        return t;
-    }
-    bool matrix(const std::string& name, uint64_t n_out, uint64_t n_in, it_weights* w) {
-        const its::Tensor* t = need(name, {n_out, n_in});
-        if (!t) return false;
-        *w = it_weights{t->data, t->bytes, t->ty, 0, n_in, n_out};
-        return true;
-    }
-    bool vec(const std::string& name, const std::vector<uint64_t>& shape, std::vector<float>* out) {
-        const its::Tensor* t = need(name, shape);
-        if (!t) return false;
-        out->resize(t->n_elems());
-        return ith::dequantize(t->ty, t->data, t->n_elems(), out->data()) || fail("tensor " + name + ": unsupported type for a vector");
-    }
     bool load(const std::string& dir) {
         itj::Value c;
         if (!read_config(dir, &c, &err) || !file.open(dir + "/model.safetensors", &err) || !config(c)) return false;
@@ -214,9 +147,6 @@ struct Serisun : it_model {
         uint64_t v[10] = {layers.size(), nd, n_vocab, a->heads, a->kv_heads, a->dim, 0, 0, 0, 0};
         memcpy(out, v, sizeof v);
     }
-    uint64_t vocab() const override { return n_vocab; }
-    uint64_t width() const override { return nd; }
-    const it_weights& embedding() const override { return embed_w; }
     template <class F> uint64_t over_runs(F per_matrix) const {
         uint64_t n = 0;
         for (const Run& r : runs) {
@@ -236,9 +166,9 @@ struct Serisun : it_model {
     it_engine* new_engine(it_hip* be, uint64_t n_ctx, uint64_t max_batch) override;
 };
 
-struct SerisunEngine : it_engine {
+struct SerisunEngine : FolderEngine {
     Serisun* m;
-    HostBuf emb, x, q, attn, u, y, ff, last, picked;
+    HostBuf emb, x, q, attn, u, y, ff;
     std::vector<HostBuf*> buffers() override { return {&emb, &x, &q, &attn, &u, &y, &ff, &last, &picked}; }
 
     void fit(uint64_t n) {
@@ -301,7 +231,7 @@ struct SerisunEngine : it_engine {
             const Attention& a = l.a;
             it_attn_bias at{q.p(), n * a.heads * a.dim, cache.k_slab(r.slot), cache.v_slab(r.slot), n_ctx * a.k_row(), n_ctx * a.v_row(),
                             start + n, a.dim, a.vdim, round8(a.dim), round8(a.vdim), a.heads, a.kv_heads, a.scale, 1, a.slopes.data(),
-                            a.temp_coef, (uint32_t)a.temp_every};
+                            a.temp_coef, (uint32_t)a.temp_every, nullptr, 0};
             it_hip_attend_bias(be, &at, attn.p(), n * l.mixed());
             o.in = attn.p();
         } else {
@@ -324,8 +254,7 @@ struct SerisunEngine : it_engine {
         it_hip_matmul_residual(be, x.p(), n * nd, terms, l.has_mlp ? 2 : 1);
     }
 
-    // Everything of a pass up to the last layer's residual; the pass stays open
-    int layers(const uint32_t* tokens, uint64_t n, uint64_t start, uint64_t ring_index) {
+    int layers(const uint32_t* tokens, uint64_t n, uint64_t start, uint64_t ring_index) override {
         if (int rc = check_pass(tokens, n, start)) return rc;
         const uint64_t nd = m->nd;
         it_hip_begin_pass(be, n);
@@ -343,8 +272,8 @@ struct SerisunEngine : it_engine {
         len = start + n;
         return 0;
     }
-    // the final norm and the head over `rows` rows of `src`
-    void head(HostBuf& src, uint64_t rows, HostBuf& out) {
+    HostBuf& residual(uint64_t) override { return x; }
+    void head(HostBuf& src, uint64_t rows, HostBuf& out) override {
         it_group_mat g;
         memset(&g, 0, sizeof g);
         g.w = m->head;
@@ -354,46 +283,11 @@ struct SerisunEngine : it_engine {
         it_hip_norm_matmuls(be, src.p(), rows * m->nd, m->final_norm.data(), m->nd, m->eps, &g, 1);
     }
 
-    int forward(const uint32_t* tokens, uint64_t n, uint64_t start, bool want_logits, uint64_t ring_index) override {
-        if (int rc = layers(tokens, n, start, ring_index)) return rc;
-        if (n == 1) {
-            head(x, 1, logits);
-        } else {
-            last.fit(m->nd, be);
-            it_hip_gather_chunks(be, x.p(), n * m->nd, m->nd, m->nd, (n - 1) * m->nd, last.p(), m->nd);
-            head(last, 1, logits);
-        }
-        it_hip_end_pass(be);
-        if (want_logits) it_hip_host_needs(be, logits.p(), m->n_vocab);
-        if (trace) tr("result_output", 0, logits, m->n_vocab);
-        return end_pass_check(!tokens);
-    }
-    int forward_rows(const uint32_t* tokens, uint64_t n, uint64_t start, const uint32_t* rows, uint64_t n_rows, float* out) override {
-        const uint64_t nv = m->n_vocab, nd = m->nd;
-        if (n == 1) {   // the same pass whether its logits are wanted or not: one recorded graph serves both
-            if (int rc = forward(tokens, 1, start, n_rows > 0, 0)) return rc;
-            if (n_rows) memcpy(out, logits.p(), nv * sizeof(float));
-            return 0;
-        }
-        if (int rc = layers(tokens, n, start, 0)) return rc;
-        it_hip_end_pass(be);
-        const uint64_t most = std::max<uint64_t>(1, std::min<uint64_t>(256, (64ull << 20) / nv));   // rows whose logits are held at a time
-        for (uint64_t at = 0; at < n_rows; at += most) {
-            const uint64_t k = std::min(most, n_rows - at);
-            last.fit(k * nd, be);
-            picked.fit(k * nv, be);
-            it_hip_gather_rows(be, x.p(), n * nd, nd, rows + at, k, last.p(), k * nd);
-            head(last, k, picked);
-            it_hip_host_needs(be, picked.p(), k * nv);
-            memcpy(out + at * nv, picked.p(), k * nv * sizeof(float));
-        }
-        return end_pass_check(false);
-    }
 };
 
 it_engine* Serisun::new_engine(it_hip* be, uint64_t n_ctx, uint64_t) {
     SerisunEngine* e = new SerisunEngine();
-    e->m = this;
+    e->fm = e->m = this;
     for (const Run& r : runs) {
         const Layer& l = layers[r.layer];
         if (l.attention) e->cache.add_kv(n_ctx * l.a.k_row(), n_ctx * l.a.v_row());
@@ -404,18 +298,6 @@ it_engine* Serisun::new_engine(it_hip* be, uint64_t n_ctx, uint64_t) {
 }
 
 }  // namespace
-
-bool config_architecture(const std::string& dir, std::string* name, std::string* err) {
-    itj::Value c;
-    if (!read_config(dir, &c, err)) return false;
-    const itj::Value* a = c.get("architecture");
-    if (!a || a->kind != itj::Value::String) {
-        *err = dir + "/config.json: no architecture";
-        return false;
-    }
-    *name = a->str;
-    return true;
-}
 
 it_model* open_serisun(const std::string& dir, std::string* err) {
     auto m = std::make_unique<Serisun>();

@@ -52,18 +52,38 @@ class Delta(C.Structure):
 class GroupMat(C.Structure):
     _fields_ = [("w", Weights), ("up", Weights), ("out", C.c_void_p), ("out_len", c_u64), ("slab", C.c_void_p),
                 ("slab_len", c_u64), ("slab_row", c_u64), ("head_dim", c_u64), ("head_stride", c_u64), ("scale", c_f32),
-                ("_pad", c_u32)]
+                ("act", c_u32)]
 
 
 class ResTerm(C.Structure):
     _fields_ = [("w", Weights), ("inp", C.c_void_p), ("in_len", c_u64), ("scale", C.c_void_p), ("norm_w", C.c_void_p),
-                ("norm_groups", c_u64), ("eps", c_f32), ("_pad", c_u32)]
+                ("norm_groups", c_u64), ("eps", c_f32), ("norm_shared", c_u32), ("gate", C.c_void_p), ("gate_len", c_u64)]
+
+
+class AddNormed(C.Structure):
+    _fields_ = [("y", C.c_void_p), ("norm_w", C.c_void_p), ("x_new", C.c_void_p), ("eps", c_f32), ("mult", c_f32)]
+
+
+class Gla(C.Structure):
+    _fields_ = [(n, C.c_void_p) for n in ("q", "k", "v", "low")] + [(n, c_u64) for n in ("q_len", "k_len", "v_len", "low_len")] + \
+               [("a2", Weights), ("a2_b", C.c_void_p), ("heads", c_u64), ("dim", c_u64), ("vdim", c_u64), ("tau", c_f32), ("_pad", c_u32)]
+
+
+class Rope(C.Structure):
+    _fields_ = [("base", C.c_double), ("dims", c_u64)] + [(n, C.c_double) for n in ("factor", "original", "fast", "slow")]
+
+
+class AttnLatent(C.Structure):
+    _fields_ = [("q", C.c_void_p), ("kv", C.c_void_p), ("q_len", c_u64), ("kv_len", c_u64), ("kv_norm", C.c_void_p), ("slab", C.c_void_p),
+                ("slab_len", c_u64), ("uk", Weights), ("uv", Weights), ("sinks", C.c_void_p), ("gate", C.c_void_p), ("gate_len", c_u64)] + \
+               [(n, c_u64) for n in ("heads", "dim", "rot_dim", "vdim", "rank", "pos", "window")] + [("scale", c_f32), ("eps", c_f32), ("rope", Rope)]
 
 
 class AttnBias(C.Structure):
     _fields_ = [("q", C.c_void_p), ("q_len", c_u64), ("k", C.c_void_p), ("v", C.c_void_p), ("k_len", c_u64), ("v_len", c_u64)] + \
                [(n, c_u64) for n in ("n_pos", "k_dim", "v_dim", "k_stride", "v_stride", "n_head", "n_head_kv")] + \
-               [("scale", c_f32), ("sink", c_u32), ("slopes", C.c_void_p), ("temp_coef", c_f32), ("temp_every", c_u32)]
+               [("scale", c_f32), ("sink", c_u32), ("slopes", C.c_void_p), ("temp_coef", c_f32), ("temp_every", c_u32), ("sinks", C.c_void_p),
+                ("window", c_u64)]
 
 
 class Mamba2(C.Structure):
@@ -126,7 +146,8 @@ it_hip_set_prefetch it_hip_set_model_path it_hip_set_map_base it_hip_expert_cove
 it_hip_expert_counts it_hip_mean_streams it_hip_mul_rows it_hip_silu it_hip_sigmoid it_hip_mul_streams it_hip_row_dot
 it_hip_signed_sqrt_sigmoid it_hip_dilated_conv it_hip_qsa_pool it_hip_qsa_select it_hip_attend_sparse
 it_hip_norm_matmuls it_hip_matmul_residual it_hip_attend_bias it_hip_mamba2 it_hip_add_rows it_hip_gather_rows it_hip_is_f32
-it_hip_zero_slab it_engine_forward_rows""".split()
+it_hip_zero_slab it_engine_forward_rows it_hip_add_normed it_hip_add_norm_matmuls it_hip_matmul_sum it_hip_gla
+it_hip_attend_latent""".split()
 
 _lib = None
 
@@ -251,6 +272,11 @@ def lib() -> C.CDLL:
         "it_engine_forward_rows": (C.c_int, [vp, vp, u64, vp, u64, vp]),
         "it_hip_norm_matmuls": (None, [vp, vp, u64, vp, u64, f32, vp, u64]),
         "it_hip_matmul_residual": (None, [vp, vp, u64, vp, u64]),
+        "it_hip_add_norm_matmuls": (None, [vp, vp, u64, vp, vp, u64, f32, vp, u64]),
+        "it_hip_add_normed": (None, [vp, vp, u64, vp, u64]),
+        "it_hip_matmul_sum": (None, [vp, vp, u64, vp, u64]),
+        "it_hip_gla": (None, [vp, vp, vp, u64, vp, u64]),
+        "it_hip_attend_latent": (None, [vp, vp, vp, u64]),
         "it_hip_attend_bias": (None, [vp, vp, vp, u64]),
         "it_hip_mamba2": (None, [vp, vp, vp, u64, vp, u64, vp, u64, vp, u64]),
         "it_hip_add_rows": (None, [vp, vp, u64, vp, vp, u64]),
@@ -442,6 +468,23 @@ class Hip:
         a = (ResTerm * len(terms))(*terms)
         self.L.it_hip_matmul_residual(self.h, _p(x), x.size, a, len(terms))
 
+    def matmul_sum(self, out, terms: list[ResTerm]):
+        a = (ResTerm * len(terms))(*terms)
+        self.L.it_hip_matmul_sum(self.h, _p(out), out.size, a, len(terms))
+
+    def add_normed(self, x, n_in, add: AddNormed):
+        self.L.it_hip_add_normed(self.h, _p(x), x.size, C.addressof(add), n_in)
+
+    def add_norm_matmuls(self, x, add: AddNormed, norm_w, n_in, eps, mats: list[GroupMat]):
+        a = (GroupMat * len(mats))(*mats)
+        self.L.it_hip_add_norm_matmuls(self.h, _p(x), x.size, C.addressof(add), _p(norm_w), n_in, eps, a, len(mats))
+
+    def gla(self, g: Gla, state, out):
+        self.L.it_hip_gla(self.h, C.addressof(g), _p(state), state.size, _p(out), out.size)
+
+    def attend_latent(self, a: AttnLatent, out):
+        self.L.it_hip_attend_latent(self.h, C.addressof(a), _p(out), out.size)
+
     def attend_bias(self, a: AttnBias, out):
         self.L.it_hip_attend_bias(self.h, C.addressof(a), _p(out), out.size)
 
@@ -490,8 +533,8 @@ class Hip:
         self.L.it_hip_profile_begin(self.h)
 
     def profile_end(self):
-        rows = (ProfileRow * 16)()
-        n = self.L.it_hip_profile_end(self.h, rows, 16)
+        rows = (ProfileRow * 24)()
+        n = self.L.it_hip_profile_end(self.h, rows, 24)
         return [dict(name=rows[i].name.decode(), launches=int(rows[i].launches), ms=float(rows[i].ms_total),
                      bytes=int(rows[i].bytes_total)) for i in range(n)]
 
