@@ -270,6 +270,8 @@ def main():
     ap.add_argument("--serisun", metavar="SIZES", nargs="?", const="w1024,w2048,w4096", default="",
                     help="another run: prefill and decode of random-weight Serisun models of these sizes (comma-separated, default "
                          "all) beside qwen35moe models of equal size, with both designs' kernels; prints its own JSON line")
+    ap.add_argument("--nubedra", metavar="SIZES", nargs="?", const="w1024,w2048,w4096", default="",
+                    help="another run: the same of random-weight Nubedra models beside Serisun models of equal size; prints its own JSON line")
     ap.add_argument("--summarize-profile", metavar="DIR",
                     help="no run: print the profiles/ summary of the rocprofv3 outputs under DIR (trace/, pmc_FETCH_SIZE/, "
                          "pmc_WRITE_SIZE/ of --decode-only runs) and exit")
@@ -288,12 +290,16 @@ def main():
         ffn = [int(t) for t in args.ffn_tokens.split(",") if t]
         print(json.dumps({"single_op": single_ops.run(ih, seed=args.seed, exact=args.exact, ffn_tokens=ffn)}), flush=True)
         return
-    if args.serisun:
+    for design, sizes in (("serisun", args.serisun), ("nubedra", args.nubedra)):
+        if not sizes:
+            continue
         import tempfile
-        from inferred_hip import serisun_bench
+        from inferred_hip import nubedra_bench, serisun_bench
         with tempfile.TemporaryDirectory(dir=str(model_path(args).parent)) as d:
-            rows = serisun_bench.run(ih, Path(d), args.serisun.split(","), steps=args.steps, seed=args.seed)
-        print(json.dumps({"serisun": rows}), flush=True)
+            side = {"serisun": serisun_bench, "nubedra": nubedra_bench}[design]
+            rows = side.run(ih, Path(d), sizes.split(","), steps=args.steps, seed=args.seed)
+        print(json.dumps({design: rows}), flush=True)
+    if args.serisun or args.nubedra:
         return
     import torch
 

@@ -61,7 +61,14 @@ def tensor_shapes(cfg):
     return out
 
 
-def write_random(folder: Path, cfg, seed=0):
+def vector(name, n, r):
+    """A vector's (or a convolution's) random values."""
+    v, leaf = r.standard_normal(n), name.rsplit(".", 1)[-1]
+    return 1 + 0.1 * v if leaf in ("norm1", "norm", "D") or name == "final.norm" else 0.3 + 0.02 * v if leaf in ("ls1", "ls2") else \
+        -3 + v if leaf == "dt_bias" else v if leaf == "A_log" else 0.3 * v
+
+
+def write_random(folder: Path, cfg, seed=0, shapes=tensor_shapes, vector=vector):
     """config.json and model.safetensors with random bf16 weights (matrices N(0, 1 / row length), cut from one random block)."""
     folder.mkdir(parents=True, exist_ok=True)
     (folder / "config.json").write_text(json.dumps(cfg))
@@ -71,7 +78,7 @@ def write_random(folder: Path, cfg, seed=0):
     def bits(a):
         return (np.ascontiguousarray(a, np.float32).view(np.uint32) >> 16).astype("<u2")
     head, at, parts = {}, 0, []
-    for name, sh in tensor_shapes(cfg).items():
+    for name, sh in shapes(cfg).items():
         n = int(np.prod(sh))
         head[name] = {"dtype": "BF16", "shape": list(sh), "data_offsets": [at, at + 2 * n]}
         at += 2 * n
@@ -86,11 +93,7 @@ def write_random(folder: Path, cfg, seed=0):
                 for lo in range(0, n, src.size):
                     src[:min(src.size, n - lo)].tofile(f)
             else:
-                v = r.standard_normal(n)
-                leaf = name.rsplit(".", 1)[-1]
-                v = 1 + 0.1 * v if leaf in ("norm1", "norm", "D") or name == "final.norm" else 0.3 + 0.02 * v if leaf in ("ls1", "ls2") else \
-                    -3 + v if leaf == "dt_bias" else v if leaf == "A_log" else 0.3 * v
-                bits(v).tofile(f)
+                bits(vector(name, n, r)).tofile(f)
     return folder
 
 
@@ -154,6 +157,24 @@ def measure(ih, model, prompt, steps, ctx):
     return min(pre), sorted(dec)[1], p_rows, d_rows, graph, chain
 
 
+def results(ih, model, prompt, steps, ctx, work, fp32=()):
+    """What measure() found, with shares of the rooflines; `work`: operations of a prefill pass by the start of a family's name, on
+    the bf16 matrix cores but for the families in `fp32`."""
+    pre, dec, p_rows, d_rows, graph, chain = measure(ih, model, prompt, steps, ctx)
+    r = {"prefill_tok_s": round(len(prompt) / pre), "prefill_ms": round(1e3 * pre, 2), "decode_tok_s": round(1 / dec, 1),
+         "decode_ms": round(1e3 * dec, 4), "decode_weight_MB": round(model.decode_weight_bytes() / 1e6, 1),
+         "decode_hbm_share": round(model.decode_weight_bytes() / dec / HBM, 3), "launches_per_token": graph["graph_kernels"], "chains": chain["chains"]}
+    r["decode_kernels"] = [dict(name=x["name"], per_token=x["launches"] / 16, us=round(1e3 * x["ms"] / x["launches"], 2),
+                                hbm_share=round(x["bytes"] / (x["ms"] * 1e-3) / HBM, 3)) for x in d_rows]
+    r["prefill_kernels"] = [dict(name=x["name"], launches=x["launches"], ms=round(x["ms"], 3)) for x in p_rows]
+    for fam, fl in work.items():
+        for k in r["prefill_kernels"]:
+            if k["name"].startswith(fam):
+                k["tflops"] = round(fl / (k["ms"] * 1e-3) / 1e12, 1)
+                k["peak_share"] = round(k["tflops"] * 1e12 / (FP32_PEAK if fam in fp32 else BF16_PEAK), 3)
+    return r
+
+
 def run(ih, tmp: Path, sizes, prompt_len=4096, steps=256, seed=0):
     out = []
     for name in sizes:
@@ -167,19 +188,7 @@ def run(ih, tmp: Path, sizes, prompt_len=4096, steps=256, seed=0):
         ih.synth_write_gguf(gguf, qwen_config(ih, s, seed))
         for kind, path in (("serisun", ds), ("qwen35moe", gguf)):
             model = ih.Model(path)
-            pre, dec, p_rows, d_rows, graph, chain = measure(ih, model, prompt, steps, ctx)
-            r = {"prefill_tok_s": round(prompt_len / pre), "prefill_ms": round(1e3 * pre, 2), "decode_tok_s": round(1 / dec, 1),
-                 "decode_ms": round(1e3 * dec, 4), "decode_weight_MB": round(model.decode_weight_bytes() / 1e6, 1),
-                 "decode_hbm_share": round(model.decode_weight_bytes() / dec / HBM, 3), "launches_per_token": graph["graph_kernels"], "chains": chain["chains"]}
-            r["decode_kernels"] = [dict(name=x["name"], per_token=x["launches"] / 16, us=round(1e3 * x["ms"] / x["launches"], 2),
-                                        hbm_share=round(x["bytes"] / (x["ms"] * 1e-3) / HBM, 3)) for x in d_rows]
-            r["prefill_kernels"] = [dict(name=x["name"], launches=x["launches"], ms=round(x["ms"], 3)) for x in p_rows]
-            if kind == "serisun":
-                for fam, fl in flops(cfg, prompt_len, prompt_len).items():
-                    for k in r["prefill_kernels"]:
-                        if k["name"].startswith(fam):
-                            k["tflops"] = round(fl / (k["ms"] * 1e-3) / 1e12, 1)
-                            k["peak_share"] = round(k["tflops"] * 1e12 / (FP32_PEAK if fam == "mamba2" else BF16_PEAK), 3)
+            r = results(ih, model, prompt, steps, ctx, flops(cfg, prompt_len, prompt_len) if kind == "serisun" else {}, ("mamba2",))
             row[kind] = r
             model.close()
             print(f"# {name} {kind}: prefill {r['prefill_tok_s']} tok/s, decode {r['decode_tok_s']} tok/s", flush=True)

@@ -42,6 +42,11 @@ def gated_recurrence(q, k, v, a):
     return o, S
 
 
+def gated_norm(o, weight, z, eps):
+    """o [n, heads, dv]: a norm per head with one weight for all of them, then the gate."""
+    return (rms(o, eps) * weight).reshape(z.shape) * silu(z)
+
+
 def gla_mixer(h, mx, w, pre, eps):
     n, H, d, dv = h.shape[0], mx["heads"], mx["dim"], mx["vdim"]
     q = (h @ w[pre + "q"].T).reshape(n, H, d) * d ** -0.5
@@ -49,8 +54,7 @@ def gla_mixer(h, mx, w, pre, eps):
     v = (h @ w[pre + "v"].T).reshape(n, H, dv)
     z = (h @ w[pre + "a1"].T) @ w[pre + "a2"].T + w[pre + "a2.b"]
     o, _ = gated_recurrence(q, k, v, key_decay(z, mx["tau"]).reshape(n, H, d))
-    o = rms(o, eps) * w[pre + "norm"]
-    return (o.reshape(n, -1) * silu(h @ w[pre + "g"].T)) @ w[pre + "o"].T
+    return gated_norm(o, w[pre + "norm"], h @ w[pre + "g"].T, eps) @ w[pre + "o"].T
 
 
 # ---------------------------------------------------------------- latent attention
@@ -81,10 +85,11 @@ def rotate(x, pos, rot):
     return y
 
 
-def visible(n, size):
-    """[query, key]: the key lies at most size - 1 tokens back (size None: anywhere before)."""
-    d = np.arange(n)[:, None] - np.arange(n)[None, :]
-    return (d >= 0) & (d < (size if size else n))
+def visible(n, m, size):
+    """[query, key], the queries at the last n of m positions: the key lies at most size - 1 tokens back (size None: anywhere
+    before)."""
+    d = np.arange(m - n, m)[:, None] - np.arange(m)[None, :]
+    return (d >= 0) & (d < (size if size else m))
 
 
 def sink_softmax(s, sink):
@@ -94,6 +99,10 @@ def sink_softmax(s, sink):
     return e / (e.sum(axis=-1, keepdims=True) + np.exp(sink - m))
 
 
+def output_gate(z):
+    return sigmoid(z)
+
+
 def latent_kv(h, mx, w, pre, eps):
     """What a latent layer keeps of every token: the normed latent and the rotated key part."""
     y = h @ w[pre + "dkv"].T
@@ -101,26 +110,40 @@ def latent_kv(h, mx, w, pre, eps):
     return c, rotate(y[:, mx["kv_rank"]:], np.arange(h.shape[0]), mx["rot"])
 
 
+def latent_attend(q, c, kr, uk, uv, scale, size, sink):
+    """q [n, H, d + r] with its last r dimensions rotated, c [m, rank], kr [m, r], uk [H * d, rank], uv [H * dv, rank],
+    sink [H]; the queries are the last n of the m positions.  -> [n, H, dv]"""
+    n, H, _ = q.shape
+    m, r = kr.shape
+    d = q.shape[2] - r
+    k = (c @ uk.T).reshape(m, H, d)
+    v = (c @ uv.T).reshape(m, H, -1)
+    seen = visible(n, m, size)
+    out = np.zeros((n, H, v.shape[2]))
+    for i in range(H):
+        s = (q[:, i, :d] @ k[:, i].T + q[:, i, d:] @ kr.T) * scale
+        out[:, i] = sink_softmax(np.where(seen, s, -np.inf), sink[i]) @ v[:, i]
+    return out
+
+
 def latent_mixer(h, kv, mx, w, pre, eps):
-    n, H, d, r, dv = h.shape[0], mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"]
+    n, H, d, r = h.shape[0], mx["heads"], mx["dim"], mx["rot_dim"]
     c, kr = kv
     cq = rms(h @ w[pre + "dq"].T, eps) * w[pre + "dq.norm"]
     q = (cq @ w[pre + "uq"].T).reshape(n, H, d + r)
-    qn, qr = q[..., :d], rotate(q[..., d:], np.arange(n), mx["rot"])
-    k = (c @ w[pre + "uk"].T).reshape(n, H, d)
-    v = (c @ w[pre + "uv"].T).reshape(n, H, dv)
-    seen = visible(n, (mx.get("mask") or {}).get("size"))
-    gate = sigmoid(h @ w[pre + "g"].T)
-    out = np.zeros((n, H, dv))
-    for i in range(H):
-        s = (qn[:, i] @ k[:, i].T + qr[:, i] @ kr.T) * mx["scale"]
-        out[:, i] = sink_softmax(np.where(seen, s, -np.inf), w[pre + "sink"][i]) @ v[:, i] * gate[:, i:i + 1]
+    q = np.concatenate([q[..., :d], rotate(q[..., d:], np.arange(n), mx["rot"])], axis=-1)
+    out = latent_attend(q, c, kr, w[pre + "uk"], w[pre + "uv"], mx["scale"], (mx.get("mask") or {}).get("size"), w[pre + "sink"])
+    out = out * output_gate(h @ w[pre + "g"].T)[:, :, None]
     return out.reshape(n, -1) @ w[pre + "o"].T
 
 
 # ---------------------------------------------------------------- the rest
+def relu(z):
+    return np.maximum(z, 0.0)
+
+
 def feed_forward(h, w, pre):
-    return (np.maximum(h @ w[pre + "gate"].T, 0.0) * (h @ w[pre + "up"].T)) @ w[pre + "down"].T
+    return (relu(h @ w[pre + "gate"].T) * (h @ w[pre + "up"].T)) @ w[pre + "down"].T
 
 
 def forward(tokens, cfg, w, layers_out=None):

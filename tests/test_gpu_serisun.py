@@ -10,68 +10,27 @@ import numpy as np
 import pytest
 
 import serisun_ref as ref
-from serisun_util import CONFIGS, attention, config, logit_error, mamba2, weights, write
+from folder_cases import MODES, Case, backend, done, engine, feed, held
+from serisun_util import CONFIGS, attention, config, logit_error, weights, write
 
 pytestmark = pytest.mark.gpu
 ROOT = Path(__file__).resolve().parent.parent
-MODES = {"bf16": {}, "f32": {"f32": True}, "steps": {"fuse": False}}
-LIMIT = {"bf16": 2e-2, "f32": 1e-4, "steps": 2e-2}
 
 
-class Case:
-    def __init__(self, folder, cfg, seed=0, w=None):
-        import inferred_hip as ih
-        self.cfg, self.w = cfg, w if w is not None else weights(cfg, seed)
-        self.path = write(folder, cfg, self.w)
-        self.model = ih.Model(self.path)
-        self.cache = {}
-
-    def logits(self, tokens):
-        key = tuple(int(t) for t in tokens)
-        if key not in self.cache:
-            self.cache[key] = ref.forward(tokens, self.cfg, self.w)
-        return self.cache[key]
-
-    def tokens(self, n, seed=0):
-        return np.random.default_rng(seed).integers(0, self.cfg["vocab"], n)
+def new_case(folder, cfg, seed=0, w=None):
+    return Case(ref, folder, cfg, w if w is not None else weights(cfg, seed))
 
 
 @pytest.fixture(scope="module")
 def cases(tmp_path_factory):
-    return {k: Case(tmp_path_factory.mktemp("serisun") / k, c, i) for i, (k, c) in enumerate(CONFIGS.items())}
+    return {k: new_case(tmp_path_factory.mktemp("serisun") / k, c, i) for i, (k, c) in enumerate(CONFIGS.items())}
 
 
 @pytest.fixture(params=sorted(MODES))
 def be(request):
-    import inferred_hip as ih
-    b = ih.Hip(**MODES[request.param])
-    b.name, b.limit = request.param, LIMIT[request.param]
+    b = backend(request.param)
     yield b
-    err = b.take_error()
-    b.close()
-    assert err is None, err
-
-
-def engine(case, be, n_ctx, max_batch=512):
-    import inferred_hip as ih
-    return ih.Engine(case.model, be, n_ctx, max_batch)
-
-
-def feed(e, tokens, sizes):
-    """The logits of every token, fed in portions of the given sizes (the last one repeated)."""
-    out, at, k = [], 0, 0
-    while at < len(tokens):
-        c = min(sizes[min(k, len(sizes) - 1)], len(tokens) - at)
-        out.append(e.forward_rows(tokens[at:at + c], np.arange(c)))
-        at, k = at + c, k + 1
-    return np.concatenate(out)
-
-
-def held(got, want, be, what=""):
-    e = logit_error(got, want)
-    assert np.isfinite(got).all()
-    # (a norm over three channels that are all near zero multiplies a 16-bit rounding: one token in fifty may be up to four times as far)
-    assert (e > be.limit).sum() <= (max(1, len(e) // 50) if be.limit > 1e-3 else 0) and e.max() < 4 * be.limit, f"{what}: {e.max():.2e} at token {int(e.argmax())}"
+    done(b)
 
 
 @pytest.mark.parametrize("name", sorted(CONFIGS))
@@ -246,7 +205,7 @@ def test_other_tensor_types_and_errors(cases, be, tmp_path):
     import inferred_hip as ih
     cfg = CONFIGS["odd"]
     w = weights(cfg, 3)
-    c = Case(tmp_path / "m", cfg, w=w)
+    c = new_case(tmp_path / "m", cfg, w=w)
     d = write(tmp_path / "n", cfg, w, {"l1.mix.q": "F32", "l0.mix.in": "F16", "embed": "F32", "head": "F16", "l2.mlp.down": "F32", "l3.norm1": "F16"})
     m = ih.Model(d)
     t = c.tokens(70, 1)
@@ -277,7 +236,7 @@ def test_a_key_far_back_decides_the_logits(tmp_path, be):
     w["l0.mix.v"][3, 2] = 1.0
     w["l0.mix.o"][20, 3] = w["l0.mix.o"][20, 19] = 1.0
     w["head"][5, 20] = w["head"][7, 1] = 1.0
-    c = Case(tmp_path / "m", cfg, w=w)
+    c = new_case(tmp_path / "m", cfg, w=w)
     for far in (0, 1, 62, 63, 64, 65, 127, 128, 129, 200):
         t = np.full(260, 4)
         t[far], t[far + 1:] = 2, np.where(np.arange(259 - far) % 3 == 0, 1, 4)
