@@ -623,7 +623,8 @@ void it_hip_attend_latent(it_hip* be, const it_attn_latent* a, float* out, uint6
     full.k = full.v = nullptr;   // (aligned; set below)
     const bool batch = be->fuse_enabled && n > FEW && uk.fmt == W_BF16 && uv.fmt == W_BF16 && attend_bias_mfma_takes(full);
     const bool split = !batch && be->fuse_enabled && attend_shared_takes(at);
-    uint16_t *c16 = nullptr, *d16 = nullptr;
+    uint16_t *c16 = nullptr, *d16 = nullptr, *q16 = nullptr;
+    int kp = 0;
     float *qa = nullptr, *ol = nullptr, *scratch = nullptr, *d32 = nullptr;
     int n_split = 0;
     if (batch) {
@@ -632,13 +633,15 @@ void it_hip_attend_latent(it_hip* be, const it_attn_latent* a, float* out, uint6
         full.v = be->tmp_for(T_VALUES, n_keys * a->heads * full.v_stride * 2);
         if (!c16 || !full.k || !full.v || !(d16 = be->act_half_out(out, n, a->heads * a->vdim)) || !(dq = be->act_inout(a->q, a->q_len))) return;
     } else {
-        if (!(qa = (float*)be->tmp_for(T_QA, n * a->heads * kd * 4))) return;
-        if (split) {   // (splits for the whole slab: a recorded pass keeps one launch shape)
+        if (split) {
+            kp = attend_shared_q_row(at);
+            if (!(q16 = (uint16_t*)be->tmp_for(T_QA, n * a->heads * (uint64_t)kp * 2))) return;
+   // (splits for the whole slab: a recorded pass keeps one launch shape)
             n_split = attend_shared_splits(at, (int)std::min<uint64_t>(cap, INT_MAX));
             BiasAttnP few = at;
             few.n_q = (int)std::min<uint64_t>(n, FEW);
             if (!(scratch = be->scratch_f32(attend_shared_scratch_floats(few, n_split)))) return;
-        } else if (!(ol = (float*)be->tmp_for(T_OL, n * a->heads * a->rank * 4))) {
+        } else if (!(qa = (float*)be->tmp_for(T_QA, n * a->heads * kd * 4)) || !(ol = (float*)be->tmp_for(T_OL, n * a->heads * a->rank * 4))) {
             return;
         }
         if (!(d32 = be->act_out(out, out_len))) return;
@@ -652,7 +655,7 @@ void it_hip_attend_latent(it_hip* be, const it_attn_latent* a, float* out, uint6
     rec.id = OP_ATTEND_LATENT;
     be->submit(it_hip::FAM_ATTEND, seen + (a->q_len + out_len) * 4,
                sig_of(OP_ATTEND_LATENT, p.q, p.kv, p.kv_norm, p.eps, p.table, p.uk, p.uk_fmt, p.uv, p.uv_fmt, p.slab, p.slab_f32, p.gate, p.heads, p.dim,
-                      p.rot, p.n_rot, p.rank, p.vdim, p.n_tok, n == 1 ? 0 : p.pos, p.n_pos_dyn, at.scale, at.sinks, at.window, c16, full.k, full.v, qa, ol,
+                      p.rot, p.n_rot, p.rank, p.vdim, p.n_tok, n == 1 ? 0 : p.pos, p.n_pos_dyn, at.scale, at.sinks, at.window, c16, full.k, full.v, qa, q16, ol,
                       scratch, n_split, d32, d16),
                rec, [=](hipStream_t s) {
                    bool ok = true;
@@ -680,20 +683,19 @@ void it_hip_attend_latent(it_hip* be, const it_attn_latent* a, float* out, uint6
                        group_gemm_bf16(g, c16, s);
                        ok = attend_bias_batch(full, nullptr, d16, s);
                    } else if (split) {
-                       latent_prep(p, qa, s);
+                       latent_prep(p, nullptr, q16, kp, at.scale, s);
                        const int few = (int)FEW;
                        for (int t0 = 0; t0 < p.n_tok && ok; t0 += few) {
                            LatentP pt = p;
                            BiasAttnP bt = at;
                            bt.n_q = pt.n_tok = std::min(few, p.n_tok - t0);
-                           bt.q = qa + (size_t)t0 * p.heads * p.k_dim();
                            if (!bt.n_pos_dyn) bt.n_pos = p.pos + t0 + bt.n_q;
                            if (p.gate) pt.gate = p.gate + (size_t)t0 * p.heads;
-                           ok = attend_shared_split(bt, n_split, scratch, s);
+                           ok = attend_shared_split(bt, q16 + (size_t)t0 * p.heads * kp, n_split, scratch, s);
                            if (ok) latent_value(pt, bt, scratch, n_split, d32 + (size_t)t0 * p.heads * p.vdim, s);
                        }
                    } else {
-                       latent_prep(p, qa, s);
+                       latent_prep(p, qa, nullptr, 0, 1.0f, s);
                        BiasAttnP bt = at;
                        bt.q = qa;
                        attend_bias_plain(bt, ol, s);

@@ -106,12 +106,12 @@ __global__ __launch_bounds__(256) void attend_bias_plain_k(BiasAttnP a, float* _
 }
 
 // ---------------------------------------------------------------- tiles of K and V
-// HD: the larger head size rounded up to whole operands.  K rows go to LDS as stored, V transposed ([dim][key]); pieces past
-// a head's stride are zeros.
-template <int HD> struct KvTile {
+// HD, HV: the key and value sizes rounded up to whole operands.  K rows go to LDS as stored, V transposed ([dim][key]); pieces
+// past a head's stride are zeros.
+template <int HD, int HV = HD> struct KvTile {
     static constexpr int KS = HD + 8;
     static constexpr int KSEG = KT * HD / 8 / 256;
-    static constexpr int UNITS = (KT / 4) * (HD / 8);
+    static constexpr int UNITS = (KT / 4) * (HV / 8);
     static constexpr int VU = (UNITS + 255) / 256;
     uint4 rk[KSEG], rv[VU][4];
     const uint16_t *kb, *vb;
@@ -361,15 +361,18 @@ __global__ __launch_bounds__(256) void attend_bias_merge_k(BiasAttnP a, const fl
 }
 
 // ---------------------------------------------------------------- many queries
-// A block: 128 (token, head) rows of one chunk of a KV head's query heads; a wave: 32 of them.
-template <int HD>
+constexpr __host__ __device__ bool q_in_registers(int hd) { return hd <= 192; }
+// A block: 128 (token, head) rows of one chunk of a KV head's query heads; a wave: 32 of them, their operands in registers (in
+// LDS where heads are so large that the accumulators need them).
+template <int HD, int HV>
 __global__ __launch_bounds__(256) void attend_bias_batch_k(BiasAttnP a, int chunks, float* __restrict__ out32, uint16_t* __restrict__ out16) {
-    typedef KvTile<HD> Tile;
-    constexpr int KS = Tile::KS, NS = HD / 16, ND = HD / 32;
+    typedef KvTile<HD, HV> Tile;
+    constexpr int KS = Tile::KS, NS = HD / 16, ND = HV / 32;
     extern __shared__ __align__(16) uint16_t blds[];
     uint16_t* Ks = blds;                 // [64][KS]
-    uint16_t* Vt = blds + KT * KS;       // [HD][VS]
-    uint16_t* Qs = Vt + HD * VS;         // [128][KS]
+    uint16_t* Vt = blds + KT * KS;       // [HV][VS]
+    constexpr bool QREG = q_in_registers(HD);
+    uint16_t* Qs = Vt + HV * VS;         // [128][KS], or nothing
     const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int r = lane & 31, g = lane >> 5;
     const int G = a.n_head / a.n_head_kv, cw = (G + chunks - 1) / chunks, QT = 128 / cw;
@@ -382,21 +385,30 @@ __global__ __launch_bounds__(256) void attend_bias_batch_k(BiasAttnP a, int chun
     const int head = kvh * G + first + (rh < nh ? rh : 0);
     const int pos = valid ? base_pos + token : base_pos;   // (a row without a query is not stored; it sees a key at least)
     const float slope2 = a.slopes ? a.slopes[head] * LOG2E : 0.0f;
-    // the block's query rows, scaled, to LDS
-    for (int i = tid; i < 128 * (HD / 4); i += 256) {
-        const int qr = i / (HD / 4), d = i % (HD / 4) * 4, tk = qt * QT + qr / cw, hh = qr % cw;
-        const bool ok = qr / cw < QT && tk < a.n_q && hh < nh;
-        uint32_t lo = 0, hi = 0;
-        if (ok) {
-            const float s = temperature(a, base_pos + tk) * (a.scale * LOG2E);
-            const float* q = a.q + ((int64_t)tk * a.n_head + kvh * G + first + hh) * a.k_dim + d;
-            uint16_t v[4];
+    // this lane's query row, scaled: eight elements of every 16
+    h8 qf[QREG ? NS : 1];
+    {
+        const float sq = valid ? temperature(a, pos) * (a.scale * LOG2E) : 0.0f;
+        const float* q = a.q + ((int64_t)(valid ? token : 0) * a.n_head + head) * a.k_dim;
+        const bool vec = a.k_dim % 4 == 0 && (reinterpret_cast<uintptr_t>(a.q) & 15) == 0;
 #pragma unroll
-            for (int e = 0; e < 4; e++) v[e] = __builtin_bit_cast(uint16_t, (_Float16)(d + e < a.k_dim ? q[e] * s : 0.0f));
-            lo = v[0] | ((uint32_t)v[1] << 16);
-            hi = v[2] | ((uint32_t)v[3] << 16);
+        for (int s = 0; s < NS; s++) {
+            const int d = 16 * s + 8 * g;
+            float v[8];
+            if (vec) {
+                const float4 x0 = d < a.k_dim ? *(const float4*)(q + d) : make_float4(0.f, 0.f, 0.f, 0.f);
+                const float4 x1 = d + 4 < a.k_dim ? *(const float4*)(q + d + 4) : make_float4(0.f, 0.f, 0.f, 0.f);
+                v[0] = x0.x; v[1] = x0.y; v[2] = x0.z; v[3] = x0.w; v[4] = x1.x; v[5] = x1.y; v[6] = x1.z; v[7] = x1.w;
+            } else {
+#pragma unroll
+                for (int e = 0; e < 8; e++) v[e] = d + e < a.k_dim ? q[d + e] : 0.0f;
+            }
+            h8 x;
+#pragma unroll
+            for (int e = 0; e < 8; e++) x[e] = (_Float16)(v[e] * sq);
+            if constexpr (QREG) qf[s] = x;
+            else *(h8*)(Qs + row * KS + d) = x;   // (read by this wave alone)
         }
-        *(uint2*)(Qs + qr * KS + d) = make_uint2(lo, hi);
     }
     const int first_pos = base_pos + qt * QT, last_pos = base_pos + min(a.n_q, (qt + 1) * QT) - 1;
     const int n_kt = last_pos / KT + 1, kt0 = first_seen(a, first_pos) / KT, seen_by_all = first_seen(a, last_pos);
@@ -425,10 +437,12 @@ __global__ __launch_bounds__(256) void attend_bias_batch_k(BiasAttnP a, int chun
             for (int i = 0; i < 16; i++) sc[kk][i] = 0.0f;
 #pragma unroll
         for (int s = 0; s < NS; s++) {
-            const h8 qf = *(const h8*)(Qs + row * KS + 16 * s + 8 * g);
+            h8 q;
+            if constexpr (QREG) q = qf[s];
+            else q = *(const h8*)(Qs + row * KS + 16 * s + 8 * g);
 #pragma unroll
             for (int kk = 0; kk < 2; kk++)
-                sc[kk] = __builtin_amdgcn_mfma_f32_32x32x16_f16(*(const h8*)(Ks + (32 * kk + r) * KS + 16 * s + 8 * g), qf, sc[kk], 0, 0, 0);
+                sc[kk] = __builtin_amdgcn_mfma_f32_32x32x16_f16(*(const h8*)(Ks + (32 * kk + r) * KS + 16 * s + 8 * g), q, sc[kk], 0, 0, 0);
             if ((s & 3) == 3) __builtin_amdgcn_sched_barrier(0);   // a few fragments in flight: registers are short
         }
         h8 ph[4], pl[4];
@@ -489,7 +503,7 @@ int padded_head(const BiasAttnP& a) {   // 0: larger than the matrix-core kernel
     return 0;
 }
 size_t split_lds(int hd) { return ((size_t)(KT + 32) * (hd + 8) + (size_t)hd * VS) * sizeof(uint16_t); }
-size_t batch_lds(int hd) { return ((size_t)(KT + 128) * (hd + 8) + (size_t)hd * VS) * sizeof(uint16_t); }
+size_t batch_lds(int hd, int hv) { return ((size_t)(KT + (q_in_registers(hd) ? 0 : 128)) * (hd + 8) + (size_t)hv * VS) * sizeof(uint16_t); }
 template <class F> bool allow_lds(F* fn, size_t lds) {
     if (lds <= 64 * 1024) return true;
     if (hipFuncSetAttribute((const void*)fn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) == hipSuccess) return true;
@@ -546,11 +560,19 @@ bool attend_bias_batch(const BiasAttnP& a, float* out32, uint16_t* out16, hipStr
     if (!attend_bias_mfma_takes(a) || a.n_pos_dyn || !a.q || !a.k || !a.v) return false;
     const int hd = padded_head(a), G = a.n_head / a.n_head_kv, chunks = (G + 31) / 32, cw = (G + chunks - 1) / chunks, QT = 128 / cw;
     const dim3 grid((unsigned)((a.n_q + QT - 1) / QT), (unsigned)(a.n_head_kv * chunks));
-#define IT_CALL(HD)                                                                                                  \
-    if (!allow_lds(attend_bias_batch_k<HD>, batch_lds(HD))) return false;                                             \
-    hipLaunchKernelGGL(attend_bias_batch_k<HD>, grid, dim3(256), batch_lds(HD), s, a, chunks, out32, out16)
+#define IT_CALL2(HD, HV)                                                                                             \
+    do {                                                                                                             \
+        if (!allow_lds(attend_bias_batch_k<HD, HV>, batch_lds(HD, HV))) return false;                                 \
+        hipLaunchKernelGGL((attend_bias_batch_k<HD, HV>), grid, dim3(256), batch_lds(HD, HV), s, a, chunks, out32, out16); \
+        return true;                                                                                                 \
+    } while (0)
+    // (values shorter than keys: the pairs that latent attention makes of 64 + 32 and 128 + 64)
+    if (hd == 96 && a.v_dim <= 64) IT_CALL2(96, 64);
+    if (hd == 192 && a.v_dim <= 128) IT_CALL2(192, 128);
+#define IT_CALL(HD) IT_CALL2(HD, HD)
     IT_HEAD(hd, IT_CALL)
 #undef IT_CALL
+#undef IT_CALL2
     return true;
 }
 #undef IT_HEAD

@@ -50,7 +50,7 @@ IT_DEV void cache_row(const LatentP& p, int t, int64_t pos, float* red) {
 // a block: 128 latent elements of one head, 16 lanes of eight; the head's rows of uk dealt to 16 groups
 constexpr int RB = 128;
 template <int FMT, bool AL>
-__global__ __launch_bounds__(256) void latent_prep_k(LatentP p, int slices, float* __restrict__ qa) {
+__global__ __launch_bounds__(256) void latent_prep_k(LatentP p, int slices, float* __restrict__ qa, uint16_t* __restrict__ q16, int kp, float qsc) {
     __shared__ float part[16][RB + 1], red[4];
     const int tid = threadIdx.x, t = blockIdx.y;
     const int64_t pos = (p.n_pos_dyn ? *p.n_pos_dyn - p.n_tok : p.pos) + t;
@@ -74,15 +74,21 @@ __global__ __launch_bounds__(256) void latent_prep_k(LatentP p, int slices, floa
 #pragma unroll
     for (int e = 0; e < 8; e++) part[dg][(tid & 15) * 8 + e] = acc[e];
     __syncthreads();
-    float* o = qa + ((int64_t)t * p.heads + h) * p.k_dim();
+    const int64_t th = (int64_t)t * p.heads + h;
+    auto store = [&](int i, float v) {
+        if (q16) q16[th * kp + i] = it_f32_to_f16(v * qsc);
+        else qa[th * p.k_dim() + i] = v;
+    };
     if (tid < RB && r0 + tid < p.rank) {
         float v = 0.0f;
 #pragma unroll
         for (int i = 0; i < 16; i++) v += part[i][tid];
-        o[r0 + tid] = v;
+        store(r0 + tid, v);
     }
-    if (r0 == 0)
-        for (int i = tid; i < p.rot; i += 256) o[p.rank + i] = rotated(p, q + p.dim, i, pos);
+    if (r0 == 0) {
+        for (int i = tid; i < p.rot; i += 256) store(p.rank + i, rotated(p, q + p.dim, i, pos));
+        if (q16 && tid < kp - p.k_dim()) q16[th * kp + p.k_dim() + tid] = 0;
+    }
 }
 
 // ---------------------------------------------------------------- many queries
@@ -113,55 +119,87 @@ __global__ __launch_bounds__(256) void latent_keys_k(LatentP p, int first, uint1
 }
 
 // ---------------------------------------------------------------- few queries, split over rows that all heads share
-// partial of (query, head, split): [v_dim padded to 32 sums][maximum in the log2 domain][sum]
+// The partials of a call: sums [query][head][split][v_dim padded to 32], behind them [query][head][split][maximum in the log2
+// domain, sum].
+struct Partials {
+    float *sums, *ml;
+    int rp, n_split;
+    IT_DEV const float* sums_of(int64_t qh) const { return sums + qh * n_split * rp; }
+    IT_DEV float* at(int64_t qh, int split) const { return sums + (qh * n_split + split) * rp; }
+    IT_DEV float* ml_at(int64_t qh, int split) const { return ml + (qh * n_split + split) * 2; }
+};
 // A block: one query's chunk of up to 32 heads (the columns of every product), one range of keys, 32 of them at a time.  The
 // waves share the scores' sum over the elements of a row (each takes every fourth 16 of them); then each holds all scores and
-// owns the output dims 32 w .. (+ 128).  Keys, values and the scaled query are f16, a probability enters the second product
-// as an f16 pair, and the operands' layouts are those of attend_bias_split_k.
+// owns the output dims 32 w .. (+ 128).  Keys, values and the scaled query (q16, rows of kp) are f16, a probability enters the
+// second product as an f16 pair, and the operands' layouts are those of attend_bias_split_k.
+// NDW: output tiles a wave; KR: 16-byte pieces a thread moves for 32 rows.
 constexpr int KT = 32;
 constexpr int SPLIT_MAX = 256;
-template <int NDW>
-__global__ __launch_bounds__(256) void attend_shared_split_k(BiasAttnP a, int n_split, int chunks, int kp, float* __restrict__ part) {
+template <int KR> struct RowPieces {
+    uint4 r[KR];
+    int nseg, dq, dr, row0, seg0;
+    IT_DEV RowPieces(int n) : nseg(n), dq(256 / n), dr(256 % n), row0(threadIdx.x / n), seg0(threadIdx.x % n) {}
+    // f(i, row, seg) of this thread's pieces
+    template <class F> IT_DEV void each(F f) {
+        int row = row0, seg = seg0;
+#pragma unroll
+        for (int i = 0; i < KR; i++) {
+            f(i, row, seg);
+            row += dq;
+            seg += dr;
+            if (seg >= nseg) seg -= nseg, row++;
+        }
+    }
+    // `rows` rows from src on, `stride` elements apart and as long at most; zeros for the rest of 32
+    IT_DEV void fetch(const uint16_t* src, int64_t stride, int rows) {
+        each([&](int i, int row, int seg) __attribute__((always_inline)) {
+            r[i] = row < rows && seg * 8 < stride ? *(const uint4*)(src + row * stride + seg * 8) : make_uint4(0, 0, 0, 0);
+        });
+    }
+    IT_DEV void stash(uint16_t* to, int rs) {
+        each([&](int i, int row, int seg) __attribute__((always_inline)) {
+            if (row < KT) *(uint4*)(to + row * rs + seg * 8) = r[i];
+        });
+    }
+};
+template <int NDW, int KR>
+__global__ __launch_bounds__(256) void attend_shared_split_k(BiasAttnP a, const uint16_t* __restrict__ q16, int chunks, int kp, Partials part) {
     extern __shared__ __align__(16) uint16_t lds[];
-    const int RS = kp + 8, NS = kp / 16, rp = (a.v_dim + 31) & ~31, ND = rp / 32;
+    const int RS = kp + 8, NS = kp / 16, ND = part.rp / 32;
     uint16_t *Ks = lds, *Qs = lds + KT * RS;            // [32][RS] each
     float* red = (float*)(lds + 2 * KT * RS);           // [wave][16][64]
     const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), c = lane & 31, g = lane >> 5;
     const int cw = (a.n_head + chunks - 1) / chunks, h0 = (blockIdx.x % chunks) * cw, t = blockIdx.x / chunks, nh = min(cw, a.n_head - h0);
-    const int split = blockIdx.y;
+    const int split = blockIdx.y, n_split = part.n_split;
     const int pos = (a.n_pos_dyn ? *a.n_pos_dyn : a.n_pos) - a.n_q + t, n_pos = pos + 1;
     const int seen = a.window ? max(0, n_pos - a.window) : 0, kpb = max(KT, ((n_pos - seen + n_split - 1) / n_split + 15) & ~15);
     const int k0 = seen + split * kpb, k1 = min(n_pos, k0 + kpb);
-    const int64_t head_stride = (int64_t)n_split * (rp + 2);
-    float* my = part + (((int64_t)t * a.n_head + h0) * n_split + split) * (rp + 2);
+    const int64_t qh = (int64_t)t * a.n_head + h0;
     if (k0 >= k1) {
         if (tid < nh) {
-            my[tid * head_stride + rp] = -INFINITY;
-            my[tid * head_stride + rp + 1] = 0.0f;
+            float* ml = part.ml_at(qh + tid, split);
+            ml[0] = -INFINITY;
+            ml[1] = 0.0f;
         }
         return;
     }
-    const float qsc = a.scale * LOG2E;
-    for (int row = tid >> 6; row < 32; row += 4)
-        for (int d = lane; d < kp; d += 64) {
-            const float v = row < nh && d < a.k_dim ? a.q[((int64_t)t * a.n_head + h0 + row) * a.k_dim + d] * qsc : 0.0f;
-            Qs[row * RS + d] = __builtin_bit_cast(uint16_t, (_Float16)v);
-        }
+    RowPieces<KR> kr(kp / 8);
+    {
+        RowPieces<KR> qr(kp / 8);
+        qr.fetch(q16 + qh * kp, kp, nh);
+        kr.fetch((const uint16_t*)a.k + (int64_t)k0 * a.k_stride, a.k_stride, k1 - k0);
+        qr.stash(Qs, RS);
+    }
     v16f o[NDW];
 #pragma unroll
     for (int dw = 0; dw < NDW; dw++)
 #pragma unroll
         for (int i = 0; i < 16; i++) o[dw][i] = 0.0f;
     float m = -INFINITY, l = 0.0f;
-    const int nseg = kp / 8;
     for (int key0 = k0; key0 < k1; key0 += KT) {
-        __syncthreads();   // the rows before are read
-        for (int row = tid >> 6; row < KT; row += 4) {
-            const uint16_t* src = (const uint16_t*)a.k + (int64_t)(key0 + row) * a.k_stride;
-            for (int seg = lane; seg < nseg; seg += 64)
-                *(uint4*)(Ks + row * RS + seg * 8) = key0 + row < k1 && seg * 8 < a.k_stride ? *(const uint4*)(src + seg * 8) : make_uint4(0, 0, 0, 0);
-        }
+        kr.stash(Ks, RS);
         __syncthreads();
+        if (key0 + KT < k1) kr.fetch((const uint16_t*)a.k + (int64_t)(key0 + KT) * a.k_stride, a.k_stride, k1 - key0 - KT);
         v16f sc;
 #pragma unroll
         for (int i = 0; i < 16; i++) sc[i] = 0.0f;
@@ -209,41 +247,51 @@ __global__ __launch_bounds__(256) void attend_shared_split_k(BiasAttnP a, int n_
                 }
             }
         }
+        __syncthreads();   // the rows are read: the next ones may land
     }
     l += __shfl_xor(l, 32, 64);
     if (c >= nh) return;
-    float* p = my + c * head_stride;
+    float* p = part.at(qh + c, split);
 #pragma unroll
     for (int dw = 0; dw < NDW; dw++) {
         const int dt = w + 4 * dw;
         if (dt < ND) {
 #pragma unroll
-            for (int i4 = 0; i4 < 4; i4++) {
-                float* q = p + 32 * dt + 8 * i4 + 4 * g;   // 8-byte aligned: the partial's size is even
-                *(float2*)q = make_float2(o[dw][4 * i4], o[dw][4 * i4 + 1]);
-                *(float2*)(q + 2) = make_float2(o[dw][4 * i4 + 2], o[dw][4 * i4 + 3]);
-            }
+            for (int i4 = 0; i4 < 4; i4++)
+                *(float4*)(p + 32 * dt + 8 * i4 + 4 * g) = make_float4(o[dw][4 * i4], o[dw][4 * i4 + 1], o[dw][4 * i4 + 2], o[dw][4 * i4 + 3]);
         }
     }
     if (w == 0 && g == 0) {
-        p[rp] = m;
-        p[rp + 1] = l;
+        float* ml = part.ml_at(qh + c, split);
+        ml[0] = m;
+        ml[1] = l;
     }
 }
 
 // ---------------------------------------------------------------- the values' matrix, behind the merge
-// a block: 32 output dims of one (query, head), a wave eight of them, four at a time
+// A block: 32 output dims of one (query, head), a wave eight of them, whose first weights are on their way while the partials
+// are merged: four elements a thread, the splits dealt to as many groups of threads as there are.
 template <int FMT, bool AL>
-__global__ __launch_bounds__(256) void latent_value_k(LatentP p, BiasAttnP a, const float* __restrict__ part, int n_split, float* __restrict__ out) {
-    extern __shared__ __align__(16) float ol[];   // [rank padded to 8]
+__global__ __launch_bounds__(256) void latent_value_k(LatentP p, BiasAttnP a, Partials part, const float* __restrict__ whole, float* __restrict__ out) {
+    extern __shared__ __align__(16) float ol[];   // [rank padded to 32], behind it [group][rank padded to 32]
     __shared__ float wsplit[SPLIT_MAX], red[8];
     __shared__ int seen;
     const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int h = blockIdx.x % p.heads;
-    if (n_split) {
-        const int rp = (p.rank + 31) & ~31, st = rp + 2;
-        const float* q = part + (int64_t)blockIdx.x * n_split * st;
-        const float ms = tid < n_split ? q[(int64_t)tid * st + rp] : -INFINITY, ls = tid < n_split ? q[(int64_t)tid * st + rp + 1] : 0.0f;
+    const int h = blockIdx.x % p.heads, j0 = blockIdx.y * 32 + w * 8;
+    const uint8_t* row[8];
+    Raw8<FMT> first[8];
+#pragma unroll
+    for (int i = 0; i < 8; i++) {
+        row[i] = row_at<FMT>(p.uv, (int64_t)h * p.vdim + min(j0 + i, p.vdim - 1), p.rank);
+        first[i] = load8<FMT, AL>(row[i], lane * 8, p.rank);
+    }
+    const float gate = p.gate ? sigmoid_exact(p.gate[blockIdx.x]) : 1.0f;
+    const int rp = (p.rank + 31) & ~31;
+    if (whole) {
+        for (int r = tid; r < rp; r += 256) ol[r] = r < p.rank ? whole[(int64_t)blockIdx.x * p.rank + r] : 0.0f;
+    } else {
+        const float* ml = part.ml_at(blockIdx.x, tid);
+        const float ms = tid < part.n_split ? ml[0] : -INFINITY, ls = tid < part.n_split ? ml[1] : 0.0f;
         float m = group_max<64>(ms);
         if (tid == 0) seen = 0;
         if (lane == 0) red[4 + w] = m;
@@ -254,44 +302,53 @@ __global__ __launch_bounds__(256) void latent_value_k(LatentP p, BiasAttnP a, co
         wsplit[tid] = wgt;
         float l = block_sum(ls * wgt, red);
         if (a.sink) l += __builtin_amdgcn_exp2f((a.sinks ? a.sinks[h] * LOG2E : 0.0f) - m);
-        const int n = seen;
-        for (int r = tid; r < pad8(p.rank); r += 256) {
-            float acc = 0.0f;
-            if (r < p.rank) {
-#pragma unroll 8
-                for (int s = 0; s < n; s++) acc = fmaf(q[(int64_t)s * st + r], wsplit[s], acc);
+        const int n = seen, r4 = rp / 4, groups = 256 / r4, grp = tid / r4;   // (rank is 1024 at most)
+        const float* q = part.sums_of(blockIdx.x) + (tid % r4) * 4;
+        float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (grp < groups) {
+#pragma unroll 16
+            for (int s = grp; s < n; s += groups) {
+                const float4 v = *(const float4*)(q + (int64_t)s * rp);
+                const float x = wsplit[s];
+                acc = make_float4(fmaf(v.x, x, acc.x), fmaf(v.y, x, acc.y), fmaf(v.z, x, acc.z), fmaf(v.w, x, acc.w));
             }
-            ol[r] = acc / l;
+            *(float4*)(ol + rp + grp * rp + (tid % r4) * 4) = acc;
         }
-    } else {
-        for (int r = tid; r < pad8(p.rank); r += 256) ol[r] = r < p.rank ? part[(int64_t)blockIdx.x * p.rank + r] : 0.0f;
+        __syncthreads();
+        for (int r = tid; r < rp; r += 256) {
+            float v = 0.0f;
+            for (int i = 0; i < groups; i++) v += ol[rp + i * rp + r];
+            ol[r] = v / l;
+        }
     }
     __syncthreads();
-    const float gate = p.gate ? sigmoid_exact(p.gate[blockIdx.x]) : 1.0f;
+    float acc[8];
 #pragma unroll
-    for (int half = 0; half < 2; half++) {
-        const int j0 = blockIdx.y * 32 + w * 8 + half * 4;
-        float acc[4] = {0.f, 0.f, 0.f, 0.f};
-        for (int k = lane * 8; k < p.rank; k += 512) {
-            const float4 x0 = *(const float4*)(ol + k), x1 = *(const float4*)(ol + k + 4);
-            const float x[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
+    for (int i = 0; i < 8; i++) acc[i] = 0.0f;
+    for (int k = lane * 8; k < p.rank; k += 512) {
+        const float4 x0 = *(const float4*)(ol + k), x1 = *(const float4*)(ol + k + 4);
+        const float x[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
 #pragma unroll
-            for (int i = 0; i < 4; i++) {
-                float f[8];
-                widen8<FMT>(load8<FMT, AL>(row_at<FMT>(p.uv, (int64_t)h * p.vdim + min(j0 + i, p.vdim - 1), p.rank), k, p.rank), f);
+        for (int i = 0; i < 8; i++) {
+            float f[8];
+            widen8<FMT>(k < 512 ? first[i] : load8<FMT, AL>(row[i], k, p.rank), f);
 #pragma unroll
-                for (int e = 0; e < 8; e++) acc[i] = fmaf(f[e], x[e], acc[i]);
-            }
+            for (int e = 0; e < 8; e++) acc[i] = fmaf(f[e], x[e], acc[i]);
         }
+    }
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            acc[i] = group_sum<64>(acc[i]);
-            if (lane == i && j0 + i < p.vdim) out[(int64_t)blockIdx.x * p.vdim + j0 + i] = acc[i] * gate;
-        }
+    for (int i = 0; i < 8; i++) {
+        acc[i] = group_sum<64>(acc[i]);
+        if (lane == i && j0 + i < p.vdim) out[(int64_t)blockIdx.x * p.vdim + j0 + i] = acc[i] * gate;
     }
 }
 
 int padded_row(const BiasAttnP& a) { return (a.k_dim + 15) & ~15; }
+Partials partials_of(const BiasAttnP& a, float* scratch, int n_split) {
+    Partials p{scratch, nullptr, (a.v_dim + 31) & ~31, n_split};
+    p.ml = scratch + (size_t)a.n_q * a.n_head * n_split * p.rp;
+    return p;
+}
 size_t shared_lds(const BiasAttnP& a) { return (size_t)2 * KT * (padded_row(a) + 8) * sizeof(uint16_t) + 4 * 16 * 64 * sizeof(float); }
 template <class F> bool allow_lds(F* fn, size_t lds) {
     if (lds <= 64 * 1024) return true;
@@ -302,11 +359,11 @@ template <class F> bool allow_lds(F* fn, size_t lds) {
 
 }  // namespace
 
-void latent_prep(const LatentP& p, float* qa, hipStream_t s) {
+void latent_prep(const LatentP& p, float* qa, uint16_t* q16, int kp, float scale, hipStream_t s) {
     const bool al = p.rank % 8 == 0 && aligned16(p.uk);
     const int slices = (p.rank + RB - 1) / RB;
     const dim3 grid(p.heads * slices + (p.kv ? 1 : 0), p.n_tok);
-#define IT_CALL(F, A) hipLaunchKernelGGL((latent_prep_k<F, A>), grid, dim3(256), 0, s, p, slices, qa)
+#define IT_CALL(F, A) hipLaunchKernelGGL((latent_prep_k<F, A>), grid, dim3(256), 0, s, p, slices, qa, q16, kp, scale * LOG2E)
     IT_BY_FORMAT(p.uk_fmt, al, IT_CALL);
 #undef IT_CALL
 }
@@ -317,8 +374,10 @@ void latent_keys(const LatentP& p, int first, int n_keys, uint16_t* c16, uint16_
 void latent_value(const LatentP& p, const BiasAttnP& a, const float* part, int n_split, float* out, hipStream_t s) {
     const bool al = p.rank % 8 == 0 && aligned16(p.uv);
     const dim3 grid(p.n_tok * p.heads, (p.vdim + 31) / 32);
-    const size_t lds = pad8(p.rank) * sizeof(float);
-#define IT_CALL(F, A) hipLaunchKernelGGL((latent_value_k<F, A>), grid, dim3(256), lds, s, p, a, part, n_split, out)
+    const int rp = (p.rank + 31) & ~31;
+    const size_t lds = (size_t)(n_split ? rp + 256 / (rp / 4) * rp : rp) * sizeof(float);   // 20 KB at most
+    const Partials pt = n_split ? partials_of(a, (float*)part, n_split) : Partials{};
+#define IT_CALL(F, A) hipLaunchKernelGGL((latent_value_k<F, A>), grid, dim3(256), lds, s, p, a, pt, n_split ? nullptr : part, out)
     IT_BY_FORMAT(p.uv_fmt, al, IT_CALL);
 #undef IT_CALL
 }
@@ -326,31 +385,33 @@ void latent_value(const LatentP& p, const BiasAttnP& a, const float* part, int n
 // one row for all heads, the values its first elements; rows of whole 16-byte pieces; no bias, no temperature
 bool attend_shared_takes(const BiasAttnP& a) {
     return !a.kv_f32 && a.k == a.v && a.n_head_kv == 1 && a.v_dim <= a.k_dim && a.k_stride % 8 == 0 && a.k_dim <= a.k_stride && !a.slopes &&
-           a.temp_coef == 0.0f && aligned16(a.k) && a.v_dim <= 1024 && shared_lds(a) <= 156 * 1024;
+           a.temp_coef == 0.0f && aligned16(a.k) && a.v_dim <= 1024 && a.k_dim <= 1088 && shared_lds(a) <= 156 * 1024;
 }
 int attend_shared_splits(const BiasAttnP& a, int n_pos_max) {
     const int most = a.window ? std::min(a.window, n_pos_max) : n_pos_max;
     return std::max(1, std::min(SPLIT_MAX, (most + 63) / 64));
 }
+int attend_shared_q_row(const BiasAttnP& a) { return padded_row(a); }
 size_t attend_shared_scratch_floats(const BiasAttnP& a, int n_split) {
     return (size_t)a.n_q * a.n_head * n_split * (((a.v_dim + 31) & ~31) + 2);
 }
-bool attend_shared_split(const BiasAttnP& a, int n_split, float* scratch, hipStream_t s) {
-    if (!attend_shared_takes(a) || n_split < 1 || n_split > SPLIT_MAX || !a.q || !a.k) return false;
-    const int chunks = (a.n_head + 31) / 32, ndw = (((a.v_dim + 31) / 32) + 3) / 4, kp = padded_row(a);
+bool attend_shared_split(const BiasAttnP& a, const uint16_t* q16, int n_split, float* scratch, hipStream_t s) {
+    if (!attend_shared_takes(a) || n_split < 1 || n_split > SPLIT_MAX || !q16 || !a.k || !scratch) return false;
+    const int chunks = (a.n_head + 31) / 32, ndw = (((a.v_dim + 31) / 32) + 3) / 4, kp = padded_row(a), kr = (KT * (kp / 8) + 255) / 256;
     const size_t lds = shared_lds(a);
     const dim3 grid((unsigned)(a.n_q * chunks), n_split);
-#define IT_CALL(N)                                                                                                        \
+    const Partials pt = partials_of(a, scratch, n_split);
+#define IT_CALL(N, R)                                                                                                     \
     do {                                                                                                                  \
-        if (!allow_lds(attend_shared_split_k<N>, lds)) return false;                                                       \
-        hipLaunchKernelGGL(attend_shared_split_k<N>, grid, dim3(256), lds, s, a, n_split, chunks, kp, scratch);            \
+        if (!allow_lds(attend_shared_split_k<N, R>, lds)) return false;                                                    \
+        hipLaunchKernelGGL((attend_shared_split_k<N, R>), grid, dim3(256), lds, s, a, q16, chunks, kp, pt);                \
+        return true;                                                                                                      \
     } while (0)
-    if (ndw <= 1) IT_CALL(1);
-    else if (ndw <= 2) IT_CALL(2);
-    else if (ndw <= 4) IT_CALL(4);
-    else IT_CALL(8);
+    if (ndw <= 1 && kr <= 3) IT_CALL(1, 3);
+    if (ndw <= 2 && kr <= 5) IT_CALL(2, 5);
+    if (ndw <= 4 && kr <= 9) IT_CALL(4, 9);
+    IT_CALL(8, 17);   // (1088 elements: what the LDS holds)
 #undef IT_CALL
-    return true;
 }
 
 }  // namespace itk

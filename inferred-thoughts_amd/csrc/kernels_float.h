@@ -199,8 +199,9 @@ struct LatentP {
     const int* n_pos_dyn;       // one token: the context's length (position + 1)
     __host__ __device__ int k_dim() const { return rank + rot; }
 };
-// queries against the latent itself: qa [token][heads][rank + rot] = [uk^T q | rotated q]; the tokens' cache rows
-void latent_prep(const LatentP& p, float* qa, hipStream_t s);
+// queries against the latent itself, [uk^T q | rotated q] of [token][heads]: f32 rows of rank + rot (qa), or f16 rows of kp, times
+// scale * log2 e and with zeros behind (q16); and the tokens' cache rows
+void latent_prep(const LatentP& p, float* qa, uint16_t* q16, int kp, float scale, hipStream_t s);
 // many tokens: their cache rows, and the rotated parts of q in place
 void latent_rows(const LatentP& p, float* q, hipStream_t s);
 // cache rows `first` .. as bf16 latents of pad8(rank) and as the rotated part of every head's key rows (f16, ks elements a head)
@@ -211,6 +212,7 @@ void latent_value(const LatentP& p, const BiasAttnP& a, const float* part, int n
 bool attend_shared_takes(const BiasAttnP& a);
 int attend_shared_splits(const BiasAttnP& a, int n_pos_max);
 size_t attend_shared_scratch_floats(const BiasAttnP& a, int n_split);
-bool attend_shared_split(const BiasAttnP& a, int n_split, float* scratch, hipStream_t s);
+int attend_shared_q_row(const BiasAttnP& a);   // elements of a row of q16
+bool attend_shared_split(const BiasAttnP& a, const uint16_t* q16, int n_split, float* scratch, hipStream_t s);   // (a.q is not read)
 
 }  // namespace itk
