@@ -633,6 +633,7 @@ void it_hip_attend_latent(it_hip* be, const it_attn_latent* a, float* out, uint6
         full.v = be->tmp_for(T_VALUES, n_keys * a->heads * full.v_stride * 2);
         if (!c16 || !full.k || !full.v || !(d16 = be->act_half_out(out, n, a->heads * a->vdim)) || !(dq = be->act_inout(a->q, a->q_len))) return;
     } else {
+        if (!(ol = (float*)be->tmp_for(T_OL, (split ? std::min<uint64_t>(n, FEW) : n) * a->heads * a->rank * 4))) return;
         if (split) {
             kp = attend_shared_q_row(at);
             if (!(q16 = (uint16_t*)be->tmp_for(T_QA, n * a->heads * (uint64_t)kp * 2))) return;
@@ -641,7 +642,7 @@ void it_hip_attend_latent(it_hip* be, const it_attn_latent* a, float* out, uint6
             BiasAttnP few = at;
             few.n_q = (int)std::min<uint64_t>(n, FEW);
             if (!(scratch = be->scratch_f32(attend_shared_scratch_floats(few, n_split)))) return;
-        } else if (!(qa = (float*)be->tmp_for(T_QA, n * a->heads * kd * 4)) || !(ol = (float*)be->tmp_for(T_OL, n * a->heads * a->rank * 4))) {
+        } else if (!(qa = (float*)be->tmp_for(T_QA, n * a->heads * kd * 4))) {
             return;
         }
         if (!(d32 = be->act_out(out, out_len))) return;
@@ -691,15 +692,15 @@ void it_hip_attend_latent(it_hip* be, const it_attn_latent* a, float* out, uint6
                            bt.n_q = pt.n_tok = std::min(few, p.n_tok - t0);
                            if (!bt.n_pos_dyn) bt.n_pos = p.pos + t0 + bt.n_q;
                            if (p.gate) pt.gate = p.gate + (size_t)t0 * p.heads;
-                           ok = attend_shared_split(bt, q16 + (size_t)t0 * p.heads * kp, n_split, scratch, s);
-                           if (ok) latent_value(pt, bt, scratch, n_split, d32 + (size_t)t0 * p.heads * p.vdim, s);
+                           ok = attend_shared_split(bt, q16 + (size_t)t0 * p.heads * kp, n_split, scratch, ol, s);
+                           if (ok) latent_value(pt, ol, d32 + (size_t)t0 * p.heads * p.vdim, s);
                        }
                    } else {
                        latent_prep(p, qa, nullptr, 0, 1.0f, s);
                        BiasAttnP bt = at;
                        bt.q = qa;
                        attend_bias_plain(bt, ol, s);
-                       latent_value(p, bt, ol, 0, d32, s);
+                       latent_value(p, ol, d32, s);
                    }
                    if (!ok) be->fail("attend_latent: the matrix-core kernels could not be launched");
                });

@@ -3,7 +3,7 @@
 //
 //   few queries:  (q_n . uk_h c) = (uk_h^T q_n) . c, so the queries are taken to the latent's space (latent_prep_k), attend to
 //       the rows as they are cached, the row's first `rank` elements being the values (attend_shared_split_k, or
-//       attend_bias_plain_k), and uv_h is applied to the sum (latent_value_k).  A row is read once for all heads.
+//       attend_bias_plain_k), and uv_h is applied to the outcome (latent_value_k).  A row is read once for all heads.
 //   many queries: the visible rows become keys and values of every head (latent_keys_k and two matrix products), which
 //       attend_bias_batch_k takes.
 //
@@ -22,6 +22,7 @@ namespace {
 typedef _Float16 h8 __attribute__((ext_vector_type(8)));
 typedef float v16f __attribute__((ext_vector_type(16)));
 constexpr float LOG2E = 1.4426950408889634f;
+constexpr int RANK_MAX = 4096;
 
 IT_DEV void slab_store(const LatentP& p, int64_t at, float v) {
     if (p.slab_f32) ((float*)p.slab)[at] = v;
@@ -268,14 +269,52 @@ __global__ __launch_bounds__(256) void attend_shared_split_k(BiasAttnP a, const 
     }
 }
 
-// ---------------------------------------------------------------- the values' matrix, behind the merge
-// A block: 32 output dims of one (query, head), a wave eight of them, whose first weights are on their way while the partials
-// are merged: four elements a thread, the splits dealt to as many groups of threads as there are.
+// One block per (query, head, 64 elements): 16 groups of threads over the splits, every one's first pieces in flight before it is
+// known which splits hold anything
+constexpr int EARLY = 8;
+__global__ __launch_bounds__(256) void attend_shared_merge_k(BiasAttnP a, Partials part, float* __restrict__ out) {
+    __shared__ float wsplit[SPLIT_MAX], red[8], sums[16][64];
+    __shared__ int seen[4];
+    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, grp = tid >> 4, r = blockIdx.y * 64 + (tid & 15) * 4;
+    const float* q = part.sums_of(blockIdx.x) + min(r, part.rp - 4);
+    float4 v[EARLY];
+#pragma unroll
+    for (int i = 0; i < EARLY; i++) v[i] = grp + 16 * i < part.n_split ? *(const float4*)(q + (int64_t)(grp + 16 * i) * part.rp) : make_float4(0.f, 0.f, 0.f, 0.f);
+    const bool has = tid < part.n_split;
+    const float* ml = part.ml_at(blockIdx.x, has ? tid : 0);
+    const float ms = has ? ml[0] : -INFINITY, ls = has ? ml[1] : 0.0f;
+    float m = group_max<64>(ms);
+    const int live = __popcll(__ballot(ms != -INFINITY));   // the splits with keys come first
+    if (lane == 0) red[4 + w] = m, seen[w] = live;
+    __syncthreads();
+    m = fmaxf(fmaxf(red[4], red[5]), fmaxf(red[6], red[7]));
+    const int n = (seen[0] + seen[1]) + (seen[2] + seen[3]), h = blockIdx.x % a.n_head;
+    const float wgt = ms != -INFINITY ? __builtin_amdgcn_exp2f(ms - m) : 0.0f;
+    wsplit[tid] = wgt;
+    float l = block_sum(ls * wgt, red);
+    if (a.sink) l += __builtin_amdgcn_exp2f((a.sinks ? a.sinks[h] * LOG2E : 0.0f) - m);
+    float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+    auto add = [&](const float4& v, float x) { acc = make_float4(fmaf(v.x, x, acc.x), fmaf(v.y, x, acc.y), fmaf(v.z, x, acc.z), fmaf(v.w, x, acc.w)); };
+#pragma unroll
+    for (int i = 0; i < EARLY; i++)
+        if (grp + 16 * i < n) add(v[i], wsplit[grp + 16 * i]);
+#pragma unroll 8
+    for (int s = grp + 16 * EARLY; s < n; s += 16) add(*(const float4*)(q + (int64_t)s * part.rp), wsplit[s]);
+    *(float4*)(&sums[grp][(tid & 15) * 4]) = acc;
+    __syncthreads();
+    if (tid < 64 && (int)blockIdx.y * 64 + tid < a.v_dim) {
+        float t = 0.0f;
+#pragma unroll
+        for (int i = 0; i < 16; i++) t += sums[i][tid];
+        out[(int64_t)blockIdx.x * a.v_dim + blockIdx.y * 64 + tid] = t / l;
+    }
+}
+
+// ---------------------------------------------------------------- the values' matrix
+// A block: 32 output dims of one (query, head), a wave eight of them
 template <int FMT, bool AL>
-__global__ __launch_bounds__(256) void latent_value_k(LatentP p, BiasAttnP a, Partials part, const float* __restrict__ whole, float* __restrict__ out) {
-    extern __shared__ __align__(16) float ol[];   // [rank padded to 32], behind it [group][rank padded to 32]
-    __shared__ float wsplit[SPLIT_MAX], red[8];
-    __shared__ int seen;
+__global__ __launch_bounds__(256) void latent_value_k(LatentP p, const float* __restrict__ ol, float* __restrict__ out) {
+    __shared__ __align__(16) float xs[RANK_MAX];
     const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int h = blockIdx.x % p.heads, j0 = blockIdx.y * 32 + w * 8;
     const uint8_t* row[8];
@@ -286,47 +325,13 @@ __global__ __launch_bounds__(256) void latent_value_k(LatentP p, BiasAttnP a, Pa
         first[i] = load8<FMT, AL>(row[i], lane * 8, p.rank);
     }
     const float gate = p.gate ? sigmoid_exact(p.gate[blockIdx.x]) : 1.0f;
-    const int rp = (p.rank + 31) & ~31;
-    if (whole) {
-        for (int r = tid; r < rp; r += 256) ol[r] = r < p.rank ? whole[(int64_t)blockIdx.x * p.rank + r] : 0.0f;
-    } else {
-        const float* ml = part.ml_at(blockIdx.x, tid);
-        const float ms = tid < part.n_split ? ml[0] : -INFINITY, ls = tid < part.n_split ? ml[1] : 0.0f;
-        float m = group_max<64>(ms);
-        if (tid == 0) seen = 0;
-        if (lane == 0) red[4 + w] = m;
-        __syncthreads();
-        m = fmaxf(fmaxf(red[4], red[5]), fmaxf(red[6], red[7]));
-        const float wgt = ms != -INFINITY ? __builtin_amdgcn_exp2f(ms - m) : 0.0f;
-        if (ms != -INFINITY) atomicMax(&seen, tid + 1);   // the splits with keys come first
-        wsplit[tid] = wgt;
-        float l = block_sum(ls * wgt, red);
-        if (a.sink) l += __builtin_amdgcn_exp2f((a.sinks ? a.sinks[h] * LOG2E : 0.0f) - m);
-        const int n = seen, r4 = rp / 4, groups = 256 / r4, grp = tid / r4;   // (rank is 1024 at most)
-        const float* q = part.sums_of(blockIdx.x) + (tid % r4) * 4;
-        float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (grp < groups) {
-#pragma unroll 16
-            for (int s = grp; s < n; s += groups) {
-                const float4 v = *(const float4*)(q + (int64_t)s * rp);
-                const float x = wsplit[s];
-                acc = make_float4(fmaf(v.x, x, acc.x), fmaf(v.y, x, acc.y), fmaf(v.z, x, acc.z), fmaf(v.w, x, acc.w));
-            }
-            *(float4*)(ol + rp + grp * rp + (tid % r4) * 4) = acc;
-        }
-        __syncthreads();
-        for (int r = tid; r < rp; r += 256) {
-            float v = 0.0f;
-            for (int i = 0; i < groups; i++) v += ol[rp + i * rp + r];
-            ol[r] = v / l;
-        }
-    }
+    for (int r = tid; r < pad8(p.rank); r += 256) xs[r] = r < p.rank ? ol[(int64_t)blockIdx.x * p.rank + r] : 0.0f;
     __syncthreads();
     float acc[8];
 #pragma unroll
     for (int i = 0; i < 8; i++) acc[i] = 0.0f;
     for (int k = lane * 8; k < p.rank; k += 512) {
-        const float4 x0 = *(const float4*)(ol + k), x1 = *(const float4*)(ol + k + 4);
+        const float4 x0 = *(const float4*)(xs + k), x1 = *(const float4*)(xs + k + 4);
         const float x[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
 #pragma unroll
         for (int i = 0; i < 8; i++) {
@@ -371,13 +376,10 @@ void latent_rows(const LatentP& p, float* q, hipStream_t s) { hipLaunchKernelGGL
 void latent_keys(const LatentP& p, int first, int n_keys, uint16_t* c16, uint16_t* k, int ks, hipStream_t s) {
     hipLaunchKernelGGL(latent_keys_k, dim3(n_keys), dim3(256), 0, s, p, first, c16, k, ks);
 }
-void latent_value(const LatentP& p, const BiasAttnP& a, const float* part, int n_split, float* out, hipStream_t s) {
+void latent_value(const LatentP& p, const float* ol, float* out, hipStream_t s) {
     const bool al = p.rank % 8 == 0 && aligned16(p.uv);
     const dim3 grid(p.n_tok * p.heads, (p.vdim + 31) / 32);
-    const int rp = (p.rank + 31) & ~31;
-    const size_t lds = (size_t)(n_split ? rp + 256 / (rp / 4) * rp : rp) * sizeof(float);   // 20 KB at most
-    const Partials pt = n_split ? partials_of(a, (float*)part, n_split) : Partials{};
-#define IT_CALL(F, A) hipLaunchKernelGGL((latent_value_k<F, A>), grid, dim3(256), lds, s, p, a, pt, n_split ? nullptr : part, out)
+#define IT_CALL(F, A) hipLaunchKernelGGL((latent_value_k<F, A>), grid, dim3(256), 0, s, p, ol, out)
     IT_BY_FORMAT(p.uv_fmt, al, IT_CALL);
 #undef IT_CALL
 }
@@ -389,13 +391,13 @@ bool attend_shared_takes(const BiasAttnP& a) {
 }
 int attend_shared_splits(const BiasAttnP& a, int n_pos_max) {
     const int most = a.window ? std::min(a.window, n_pos_max) : n_pos_max;
-    return std::max(1, std::min(SPLIT_MAX, (most + 63) / 64));
+    return std::max(1, std::min(most <= 8192 ? 128 : SPLIT_MAX, (most + KT - 1) / KT));
 }
 int attend_shared_q_row(const BiasAttnP& a) { return padded_row(a); }
 size_t attend_shared_scratch_floats(const BiasAttnP& a, int n_split) {
     return (size_t)a.n_q * a.n_head * n_split * (((a.v_dim + 31) & ~31) + 2);
 }
-bool attend_shared_split(const BiasAttnP& a, const uint16_t* q16, int n_split, float* scratch, hipStream_t s) {
+bool attend_shared_split(const BiasAttnP& a, const uint16_t* q16, int n_split, float* scratch, float* out, hipStream_t s) {
     if (!attend_shared_takes(a) || n_split < 1 || n_split > SPLIT_MAX || !q16 || !a.k || !scratch) return false;
     const int chunks = (a.n_head + 31) / 32, ndw = (((a.v_dim + 31) / 32) + 3) / 4, kp = padded_row(a), kr = (KT * (kp / 8) + 255) / 256;
     const size_t lds = shared_lds(a);
@@ -405,6 +407,7 @@ bool attend_shared_split(const BiasAttnP& a, const uint16_t* q16, int n_split, f
     do {                                                                                                                  \
         if (!allow_lds(attend_shared_split_k<N, R>, lds)) return false;                                                    \
         hipLaunchKernelGGL((attend_shared_split_k<N, R>), grid, dim3(256), lds, s, a, q16, chunks, kp, pt);                \
+        hipLaunchKernelGGL(attend_shared_merge_k, dim3((unsigned)(a.n_q * a.n_head), (pt.rp + 63) / 64), dim3(256), 0, s, a, pt, out); \
         return true;                                                                                                      \
     } while (0)
     if (ndw <= 1 && kr <= 3) IT_CALL(1, 3);

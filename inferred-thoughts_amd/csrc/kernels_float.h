@@ -206,13 +206,14 @@ void latent_prep(const LatentP& p, float* qa, uint16_t* q16, int kp, float scale
 void latent_rows(const LatentP& p, float* q, hipStream_t s);
 // cache rows `first` .. as bf16 latents of pad8(rank) and as the rotated part of every head's key rows (f16, ks elements a head)
 void latent_keys(const LatentP& p, int first, int n_keys, uint16_t* c16, uint16_t* k, int ks, hipStream_t s);
-// out [token][heads * vdim] = gate * uv (merged partials of attend_shared_split; n_split 0: `part` holds [token][heads][rank])
-void latent_value(const LatentP& p, const BiasAttnP& a, const float* part, int n_split, float* out, hipStream_t s);
-// few queries against rows whose first v_dim elements are the values, one row for all heads: partial sums of f16 matrix cores
+// out [token][heads * vdim] = gate * uv ol, ol [token][heads][rank]
+void latent_value(const LatentP& p, const float* ol, float* out, hipStream_t s);
+// few queries against rows whose first v_dim elements are the values, one row for all heads, on the f16 matrix cores:
+// out [query][head][v_dim]
 bool attend_shared_takes(const BiasAttnP& a);
 int attend_shared_splits(const BiasAttnP& a, int n_pos_max);
 size_t attend_shared_scratch_floats(const BiasAttnP& a, int n_split);
 int attend_shared_q_row(const BiasAttnP& a);   // elements of a row of q16
-bool attend_shared_split(const BiasAttnP& a, const uint16_t* q16, int n_split, float* scratch, hipStream_t s);   // (a.q is not read)
+bool attend_shared_split(const BiasAttnP& a, const uint16_t* q16, int n_split, float* scratch, float* out, hipStream_t s);   // (a.q is not read)
 
 }  // namespace itk
