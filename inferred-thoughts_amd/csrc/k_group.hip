@@ -406,6 +406,38 @@ __global__ __launch_bounds__(256) void norm_gate_rows_k(const float* __restrict_
     if (out16 && j0 + part == nd && lane < pad8(nd) - nd) out16[row * pad8(nd) + nd + lane] = 0;
 }
 
+// the same for parts of whole float4s, rows of whole 16-byte bf16 pieces: a lane keeps its V pieces
+template <int V>
+__global__ __launch_bounds__(256) void norm_gate_rows4_k(const float* __restrict__ x, const float* __restrict__ w, int period, const float* __restrict__ gate,
+                                                         int groups, float eps, int64_t n_parts, int nd, float* __restrict__ out32, uint16_t* __restrict__ out16) {
+    const int part = nd / groups, n4 = part >> 2, lane = threadIdx.x & 63;
+    const int64_t at = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (at >= n_parts) return;
+    const int64_t at0 = at * part;   // (rows are `groups` parts)
+    if (period != part) w += at % groups * part;
+    float4 v[V], z[V];
+    float ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < V; i++) {
+        const int k = lane + i * 64;
+        v[i] = k < n4 ? ((const float4*)(x + at0))[k] : make_float4(0.f, 0.f, 0.f, 0.f);
+        if (gate) z[i] = k < n4 ? ((const float4*)(gate + at0))[k] : make_float4(0.f, 0.f, 0.f, 0.f);
+        ss = fmaf(v[i].x, v[i].x, fmaf(v[i].y, v[i].y, fmaf(v[i].z, v[i].z, fmaf(v[i].w, v[i].w, ss))));
+    }
+    const float rinv = 1.0f / sqrtf(group_sum<64>(ss) / (float)part + eps);
+#pragma unroll
+    for (int i = 0; i < V; i++) {
+        const int k = lane + i * 64;
+        if (k >= n4) continue;
+        const float4 ww = ((const float4*)w)[k];
+        float4 r = make_float4(v[i].x * rinv * ww.x, v[i].y * rinv * ww.y, v[i].z * rinv * ww.z, v[i].w * rinv * ww.w);
+        if (gate) r = make_float4(r.x * silu_exact(z[i].x), r.y * silu_exact(z[i].y), r.z * silu_exact(z[i].z), r.w * silu_exact(z[i].w));
+        if (out32) ((float4*)(out32 + at0))[k] = r;
+        if (out16)
+            ((uint2*)(out16 + at0))[k] = make_uint2(to_bf16(r.x) | ((uint32_t)to_bf16(r.y) << 16), to_bf16(r.z) | ((uint32_t)to_bf16(r.w) << 16));
+    }
+}
+
 // V > 0: rows of whole float4s, a thread keeps its V pieces; V = 0: any row, through x_new
 template <int V>
 __global__ __launch_bounds__(256) void add_norm_rows_k(const float* __restrict__ x, AddNormed a, const float* __restrict__ w, float eps, int nd,
@@ -632,6 +664,13 @@ void norm_gate_rows(const float* x, const float* w, int period, const float* gat
                     float* out32, uint16_t* out16, hipStream_t s) {
     if (n_rows <= 0) return;
     const int64_t parts = n_rows * groups;
+    const int part = nd / groups;
+    if (nd % 8 == 0 && part % 4 == 0 && part <= 1024 && aligned16(x) && aligned16(w) && aligned16(gate) && aligned16(out32) && aligned16(out16)) {
+        const dim3 grid((unsigned)((parts + 3) / 4));
+        if (part <= 256) hipLaunchKernelGGL(norm_gate_rows4_k<1>, grid, dim3(256), 0, s, x, w, period, gate, groups, eps, parts, nd, out32, out16);
+        else hipLaunchKernelGGL(norm_gate_rows4_k<4>, grid, dim3(256), 0, s, x, w, period, gate, groups, eps, parts, nd, out32, out16);
+        return;
+    }
     hipLaunchKernelGGL(norm_gate_rows_k, dim3((unsigned)((parts + 3) / 4)), dim3(256), 0, s, x, w, period, gate, groups, eps, parts, nd, out32, out16);
 }
 

@@ -72,7 +72,7 @@ def test_a_pair_with_relu(be, n, n_in, ff):
     assert rel(read_rows(be, out, n, ff), ref.relu(h @ gate.v.T) * (h @ up.v.T)) < (3e-2 if be.name == "default" and n > 16 else 1e-2 if n > 16 and not be.f32 else 2e-5)
 
 
-@pytest.mark.parametrize("nd, heads, dv", [(64, 3, 24), (37, 5, 7), (96, 1, 130), (600, 12, 64)])
+@pytest.mark.parametrize("nd, heads, dv", [(64, 3, 24), (37, 5, 7), (96, 1, 130), (600, 12, 64), (40, 2, 300), (24, 1, 1200)])
 @pytest.mark.parametrize("gated", [True, False])
 @pytest.mark.parametrize("n", TOKENS)
 def test_a_product_of_normed_and_gated_heads(be, n, gated, nd, heads, dv):
